@@ -514,6 +514,75 @@ int llm_decoder_run_attention(llm_decoder* d, int layer, void* stream);
 int llm_decoder_context_len(const llm_decoder* d, int row);
 kv_cache* llm_decoder_kv(llm_decoder* d);
 
+/* ------------------------------------------------------------------------ */
+/* Serving engine: any registered model behind one step function, with       */
+/* sequences that come and go, mixed batches and a scheduler.                 */
+/* ------------------------------------------------------------------------ */
+typedef struct llm_engine llm_engine;
+
+typedef struct llm_engine_config {
+  int dtype;            /* LLM_BF16 (weights, products and cache in bf16) or LLM_F32 */
+  int max_seqs;         /* live sequences (cache slots) */
+  long long max_tokens; /* most tokens live sequences hold, each rounded up to whole pages */
+  int max_seq_len;      /* longest sequence; 0 -> max_tokens */
+  int max_step_tokens;  /* tokens of one forward pass; 0 -> the model's default */
+} llm_engine_config;
+
+/* Registered model architectures, comma-separated. */
+const char* llm_model_architectures(void);
+
+/* Build the model of a folder: config.json names its architecture in the
+ * registry, model.safetensors (or the architecture's own files) its weights. */
+int llm_engine_create(const char* model_dir, const llm_engine_config* cfg, llm_engine** out);
+void llm_engine_destroy(llm_engine* e);
+int llm_engine_vocab(const llm_engine* e);
+int llm_engine_max_seq_len(const llm_engine* e);
+int llm_engine_page_tokens(const llm_engine* e);
+/* Tokens the cache pool can still take in whole pages. */
+long long llm_engine_free_tokens(llm_engine* e);
+
+/* Low-level stepping.  A sequence holds a cache slot from open to close. */
+int llm_engine_open(llm_engine* e, int* seq);
+int llm_engine_close(llm_engine* e, int seq);
+int llm_engine_seq_len(llm_engine* e, int seq); /* tokens so far, -1: not open */
+typedef struct llm_engine_entry {
+  int seq;
+  const int32_t* tokens; /* its next n tokens */
+  int n;
+  const int32_t* want;   /* places among them whose logits are wanted */
+  int n_want;
+} llm_engine_entry;
+/* One step: every entry's tokens in one batch (portions of prompts beside
+ * single tokens), from what earlier steps left in the cache.  logits: host
+ * [wanted rows][vocab], in the order of the entries and of `want` (NULL only
+ * when nothing is wanted).  A failed step leaves the sequences' lengths as
+ * they were. */
+int llm_engine_step(llm_engine* e, const llm_engine_entry* entries, int n, float* logits);
+/* The residual stream after every layer run of each following step of at most
+ * max_step_tokens tokens: tap, host [layer runs][tokens][width]; NULL: off. */
+int llm_engine_set_tap(llm_engine* e, float* tap);
+int llm_engine_layer_runs(const llm_engine* e);
+int llm_engine_width(const llm_engine* e);
+
+/* Scheduler: requests wait until a slot and the pages for their whole length
+ * are free; every pass runs one token of each generating request and, in the
+ * tokens left, portions of waiting prompts. */
+typedef struct llm_request_params {
+  int max_new_tokens;
+  float temperature; /* <= 0: greedy */
+  int top_k;         /* 0: off */
+  float top_p;       /* 1: off; 0 is read as 1 */
+  uint64_t seed;     /* draws depend on (seed, position) alone */
+  int eos_token;     /* ends the request; -1: none */
+} llm_request_params;
+int llm_engine_submit(llm_engine* e, const int32_t* prompt, int n, const llm_request_params* p,
+                      int* request);
+/* One scheduler pass; *active: requests still waiting or running. */
+int llm_engine_run(llm_engine* e, int* active);
+/* Tokens generated so far (up to cap into out); a finished request whose
+ * tokens all fit is forgotten by this call. */
+int llm_engine_result(llm_engine* e, int request, int32_t* out, int cap, int* n, int* finished);
+
 #ifdef __cplusplus
 }
 #endif

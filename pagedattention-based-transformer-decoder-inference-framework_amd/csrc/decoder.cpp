@@ -29,6 +29,7 @@
 #include <vector>
 
 #include "common.hpp"
+#include "dev_buf.hpp"
 #include "gemm.hpp"
 #include "kv_cache_impl.hpp"
 #include "pa_decode.hpp"
@@ -39,30 +40,6 @@ using namespace llm;
 // f[1] = f[0], f[0] = 0 in one device atomic: the fused o_proj's range flag
 // read and cleared (llm_decoder::report_range)
 __global__ void take_flag_kernel(int* f) { f[1] = atomicExch(f, 0); }
-
-namespace {
-
-template <typename T>
-struct DevBuf {
-  T* p = nullptr;
-  size_t n = 0;
-  ~DevBuf() { if (p) (void)hipFree(p); }
-  int alloc(size_t count) {
-    if (p) { (void)hipFree(p); p = nullptr; }
-    n = count;
-    if (count == 0) return LLM_OK;
-    if (hipMalloc(&p, count * sizeof(T)) != hipSuccess) {
-      (void)hipGetLastError();
-      return fail(LLM_ERR_OOM, "decoder: device allocation of " + std::to_string(count * sizeof(T)) +
-                                   " bytes failed");
-    }
-    return LLM_OK;
-  }
-};
-
-#define RET_IF(x) do { int _rc = (x); if (_rc) return _rc; } while (0)
-
-}  // namespace
 
 struct llm_decoder {
   llm_decoder_config cfg{};

@@ -56,11 +56,13 @@ __global__ void kv_write_tokens_kernel(const E* __restrict__ ksrc, const E* __re
 }
 
 int KvCache::init(int L_, int beams_, int H_, int D_, int TS_, int max_tiles_, long long pages,
-                  int dtype_) {
+                  int dtype_, int Dv_) {
   L = L_; beams = beams_; H = H_; D = D_; TS = TS_; max_tiles = max_tiles_; num_pages = pages;
   dtype = dtype_;
   es = dtype == LLM_F32 ? 4 : dtype == LLM_I8 ? 1 : 2;
+  Dv = Dv_ > 0 ? Dv_ : D;
   page_elems = (size_t)TS * D;
+  v_page_elems = (size_t)TS * Dv;
   // A wave loads K page p and V page p together.  With two separate pools at
   // a large distance the pair often falls into the same HBM channel and the
   // scan loses 2-4 %, depending on the distance (C3 shape,
@@ -83,6 +85,12 @@ int KvCache::init(int L_, int beams_, int H_, int D_, int TS_, int max_tiles_, l
   refcount.assign((size_t)num_pages, 0);
   reset_free_lists();
   LLM_HIP_RET(hipEventCreateWithFlags(&staging_done, hipEventDisableTiming));
+  return LLM_OK;
+}
+
+int KvCache::zero_pools(hipStream_t st) {
+  LLM_HIP_RET(hipMemsetAsync(k_pool, 0, (size_t)num_pages * page_stride(), st));
+  LLM_HIP_RET(hipStreamSynchronize(st));
   return LLM_OK;
 }
 
@@ -225,6 +233,18 @@ int KvCache::prepare_append(int beam, int pos) {
       if (rc) return rc;
     }
   return LLM_OK;
+}
+
+void KvCache::release_beam(int beam) {
+  for (int l = 0; l < L; ++l)
+    for (int h = 0; h < H; ++h)
+      for (int t = 0; t < max_tiles; ++t) {
+        const size_t i = index(l, beam, h, t);
+        if (h_table[i] >= 0) {
+          drop_page(h_table[i]);
+          set_entry(i, -1);
+        }
+      }
 }
 
 int KvCache::sync(hipStream_t st) {
@@ -435,15 +455,7 @@ extern "C" int kv_cache_release(kv_cache* c, int beam) {
   KvCache& k = c->impl;
   std::lock_guard<std::mutex> g(k.mu);
   LLM_REQUIRE(beam >= 0 && beam < k.beams, "kv_cache_release: bad beam");
-  for (int l = 0; l < k.L; ++l)
-    for (int h = 0; h < k.H; ++h)
-      for (int t = 0; t < k.max_tiles; ++t) {
-        const size_t i = k.index(l, beam, h, t);
-        if (k.h_table[i] >= 0) {
-          k.drop_page(k.h_table[i]);
-          k.set_entry(i, -1);
-        }
-      }
+  k.release_beam(beam);
   return LLM_OK;
 }
 

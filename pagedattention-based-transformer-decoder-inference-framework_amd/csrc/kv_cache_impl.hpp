@@ -17,10 +17,12 @@ namespace llm {
 
 struct KvCache {
   int L = 0, beams = 0, H = 0, D = 0, TS = 0, max_tiles = 0;
+  int Dv = 0;  // value head size (D unless init was given another)
   long long num_pages = 0;
   int dtype = LLM_F16;  // pool element type
   int es = 2;           // bytes per element
-  size_t page_elems = 0;
+  size_t page_elems = 0;    // of a K page
+  size_t v_page_elems = 0;  // of a V page
   size_t entries = 0;
   void* k_pool = nullptr;  // page p of K at k_pool + p * page_stride(), V right after it
   void* v_pool = nullptr;  // = k_pool + page_bytes() (same allocation)
@@ -60,9 +62,11 @@ struct KvCache {
 
   ~KvCache();
   int init(int L, int beams, int H, int D, int TS, int max_tiles, long long pages,
-           int dtype = LLM_F16);
+           int dtype = LLM_F16, int Dv = 0);
+  // zero the pools (layouts that pad their rows rely on zero padding)
+  int zero_pools(hipStream_t st);
   size_t page_bytes() const { return page_elems * es; }
-  size_t page_stride() const { return 2 * page_bytes(); }  // K and V pages interleave
+  size_t page_stride() const { return (page_elems + v_page_elems) * es; }  // K and V pages interleave
   size_t index(int layer, int beam, int head, int tile) const {
     return (((size_t)layer * beams + beam) * H + head) * max_tiles + tile;
   }
@@ -81,6 +85,8 @@ struct KvCache {
   int ensure_tile(int layer, int beam, int head, int tile, bool exclusive, int32_t* page);
   // make the tile of `pos` exist and be exclusive for every layer / head of `beam`
   int prepare_append(int beam, int pos);
+  // give back every page of `beam`
+  void release_beam(int beam);
   // push copy-on-write copies and dirty table entries to the device (stream-ordered)
   int sync(hipStream_t st);
 };

@@ -1,0 +1,70 @@
+// Decoder-only models given as a list of layers (csrc/layer_stack.cpp): every
+// layer names its mixer and its feed-forward with sizes of their own, a run of
+// layers may repeat with the same weights, norms stand before and after each
+// sublayer.  A model family reads its config.json into LayerStackConfig.
+#pragma once
+
+#include <memory>
+#include <string>
+#include <vector>
+
+#include "mm.hpp"
+#include "model.hpp"
+
+namespace llm {
+
+// Rotary positions on the first `dims` dimensions of a head, partners half of
+// `dims` apart; with yarn the frequencies are interpolated (rope_frequencies).
+struct RopeSpec {
+  int dims = 0;
+  double base = 10000.0;
+  bool yarn = false;
+  double factor = 1.0, original = 1.0, fast = 32.0, slow = 1.0;
+  bool operator==(const RopeSpec& o) const {
+    return dims == o.dims && base == o.base && yarn == o.yarn && factor == o.factor &&
+           original == o.original && fast == o.fast && slow == o.slow;
+  }
+};
+// Frequency of each of the dims / 2 pairs; *mul: the factor on cosine and sine.
+std::vector<float> rope_frequencies(const RopeSpec& r, float* mul);
+
+struct AttentionSpec {
+  int heads = 0, kv_heads = 0, dim = 0, vdim = 0;
+  RopeSpec rope;
+  float scale = 1.f;
+  bool sink = false;  // a learned term in each head's softmax denominator
+};
+
+struct ExpertSpec {
+  int ff = 0;
+  GluParams glu;
+};
+struct MoeSpec {
+  int experts = 0, top = 0;
+  float scale = 1.f;
+  ExpertSpec expert;
+  bool has_shared = false;
+  ExpertSpec shared;
+};
+
+struct LayerSpec {
+  AttentionSpec attn;
+  bool has_mlp = false;
+  MoeSpec moe;
+};
+
+struct LayerStackConfig {
+  int vocab = 0, width = 0;
+  float eps = 1e-5f;
+  std::vector<LayerSpec> layers;
+  // layers [loop_start, loop_stop) run loop_times times in a row; each pass but
+  // the first adds the embedding output to the residual before its first layer
+  int loop_start = 0, loop_stop = 0, loop_times = 1;
+};
+
+// Checks the configuration, reads the weights of dir/model.safetensors (tensor
+// names: embed, l<i>.norm1 ..., final.norm, head) and builds the model.
+int make_layer_stack(const LayerStackConfig& cfg, const std::string& dir, const ModelOptions& opt,
+                     std::unique_ptr<StepModel>* out);
+
+}  // namespace llm

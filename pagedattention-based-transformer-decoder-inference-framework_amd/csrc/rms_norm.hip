@@ -1,0 +1,152 @@
+// The residual stream between sublayers: add the normed sublayer output, add
+// the embedding where a repeated pass starts, norm for the next sublayer --
+// one launch, the row in registers.  Also the rotation angles of a step.
+#include "common.hpp"
+#include "rms_norm.hpp"
+
+namespace llm {
+namespace {
+
+typedef __bf16 bf16x4 __attribute__((ext_vector_type(4)));
+
+template <int THREADS>
+__device__ __forceinline__ float row_sum(float v, float* sh) {
+  v = wave_sum(v);
+  if constexpr (THREADS == 64) return v;
+  __syncthreads();  // sh free again
+  if (lane_id() == 0) sh[wave_id_uniform()] = v;
+  __syncthreads();
+  float s = sh[0];
+#pragma unroll
+  for (int i = 1; i < THREADS / 64; ++i) s += sh[i];
+  return s;
+}
+
+__device__ __forceinline__ float square_sum(f32x4 v) {
+  return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+}
+
+// THREADS lanes per row, NV float4 per lane
+template <typename T, int THREADS, int NV>
+__global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
+  __shared__ float sh[THREADS / 64];
+  const int i = blockIdx.x;
+  const int m = a.rows ? a.rows[i] : i;
+  const int nv = a.ldx >> 2;
+  float* xr = a.x + (size_t)m * a.ldx;
+  f32x4 x[NV];
+  auto embed_at = [&](int c) {
+    const uint2 e = *reinterpret_cast<const uint2*>(a.emb + (size_t)a.tok[m] * a.ldx + 4 * c);
+    return f32x4{__builtin_bit_cast(float, e.x << 16), __builtin_bit_cast(float, e.x & 0xFFFF0000u),
+                 __builtin_bit_cast(float, e.y << 16), __builtin_bit_cast(float, e.y & 0xFFFF0000u)};
+  };
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * THREADS;
+    x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < nv) x[j] = a.embed == 1 ? embed_at(c) : *reinterpret_cast<const f32x4*>(xr + 4 * c);
+  }
+  const float inv_w = 1.f / (float)a.width;
+  if (a.w_post) {
+    f32x4 y[NV];
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = threadIdx.x + j * THREADS;
+      f32x4 s = {0.f, 0.f, 0.f, 0.f};
+      if (c < nv) {
+        for (int q = 0; q < a.parts; ++q)
+          s += *reinterpret_cast<const f32x4*>(a.y + ((size_t)m * a.parts + q) * a.ldy + 4 * c);
+        if (a.shared)
+          s += *reinterpret_cast<const f32x4*>(a.y + ((size_t)a.M_y * a.parts + m) * a.ldy + 4 * c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e)
+          if (4 * c + e >= a.width) s[e] = 0.f;
+      }
+      y[j] = s;
+      ss += square_sum(s);
+    }
+    const float r = 1.f / sqrtf(row_sum<THREADS>(ss, sh) * inv_w + a.eps);
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = threadIdx.x + j * THREADS;
+      if (c < nv) x[j] += y[j] * r * *reinterpret_cast<const f32x4*>(a.w_post + 4 * c);
+    }
+  }
+  if (a.embed == 2) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = threadIdx.x + j * THREADS;
+      if (c < nv) x[j] += embed_at(c);
+    }
+  }
+  if ((a.w_post || a.embed) && !a.rows) {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) {
+      const int c = threadIdx.x + j * THREADS;
+      if (c < nv) *reinterpret_cast<f32x4*>(xr + 4 * c) = x[j];
+    }
+  }
+  if (!a.w_pre) return;
+  float ss = 0.f;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) ss += square_sum(x[j]);
+  const float r = 1.f / sqrtf(row_sum<THREADS>(ss, sh) * inv_w + a.eps);
+  T* hr = static_cast<T*>(a.h) + (size_t)i * a.ldh;
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * THREADS;
+    if (c >= nv) continue;
+    const f32x4 o = x[j] * r * *reinterpret_cast<const f32x4*>(a.w_pre + 4 * c);
+    if constexpr (sizeof(T) == 2)
+      *reinterpret_cast<bf16x4*>(hr + 4 * c) =
+          bf16x4{(__bf16)o[0], (__bf16)o[1], (__bf16)o[2], (__bf16)o[3]};
+    else
+      *reinterpret_cast<f32x4*>(hr + 4 * c) = o;
+  }
+}
+
+template <typename T>
+hipError_t launch_norm(const NormStep& a, hipStream_t st) {
+  const dim3 grid(a.M);
+  const int nv = a.ldx >> 2;
+#define LLM_NORM_GO(TH, NV)                                                           \
+  hipLaunchKernelGGL((norm_step_kernel<T, TH, NV>), grid, dim3(TH), 0, st, a);        \
+  return hipGetLastError()
+  if (nv <= 64) { LLM_NORM_GO(64, 1); }
+  if (nv <= 128) { LLM_NORM_GO(64, 2); }
+  if (nv <= 256) { LLM_NORM_GO(256, 1); }
+  if (nv <= 512) { LLM_NORM_GO(256, 2); }
+  if (nv <= 1024) { LLM_NORM_GO(256, 4); }
+  if (nv <= 2048) { LLM_NORM_GO(256, 8); }
+#undef LLM_NORM_GO
+  return hipErrorInvalidValue;
+}
+
+__global__ void rope_turns_kernel(const int32_t* __restrict__ pos, int M,
+                                  const float* __restrict__ freq, int half, float mul,
+                                  float2* __restrict__ turn) {
+  const int idx = blockIdx.x * blockDim.x + threadIdx.x;
+  if (idx >= M * half) return;
+  const float a = (float)pos[idx / half] * freq[idx % half];
+  float s, c;
+  sincosf(a, &s, &c);
+  turn[idx] = float2{c * mul, s * mul};
+}
+
+}  // namespace
+
+hipError_t rms_norm_step(int dtype, const NormStep& a, hipStream_t st) {
+  if (a.M <= 0) return hipSuccess;
+  return dtype == LLM_F32 ? launch_norm<float>(a, st) : launch_norm<__bf16>(a, st);
+}
+
+hipError_t rope_turns(const int32_t* pos, int M, const float* freq, int half, float mul,
+                      float2* turn, hipStream_t st) {
+  if (M <= 0 || half <= 0) return hipSuccess;
+  hipLaunchKernelGGL(rope_turns_kernel, dim3((M * half + 255) / 256), dim3(256), 0, st, pos, M,
+                     freq, half, mul, turn);
+  return hipGetLastError();
+}
+
+}  // namespace llm
