@@ -32,6 +32,7 @@
 #include "dev_buf.hpp"
 #include "gemm.hpp"
 #include "kv_cache_impl.hpp"
+#include "model.hpp"
 #include "pa_decode.hpp"
 #include "row_ops.hpp"
 
@@ -148,7 +149,9 @@ struct llm_decoder {
   DevBuf<int32_t> pmeta;  // [4][chunk]: pos, ctx, page-table row, token
   size_t pws_bytes = 0;
   int pf_cap = 0;
+  int ensure_prefill(int C);
   int prefill(int row, const int32_t* toks, int n, hipStream_t st);
+  int forward_mixed(const std::vector<StepSeq>& seqs, float* logits_dev, hipStream_t st);
 };
 
 static int check_cfg(const llm_decoder_config& c) {
@@ -387,6 +390,9 @@ struct Rows {
   // row prefill_row, attended causally by the MFMA prefill kernel
   int prefill_row = -1;
   int prefill_p0 = 0;
+  // tokens of several sequences (the serving engine's step): prefill rows that
+  // take the paged decode attention, each by its own page-table row and context
+  bool mixed = false;
   uint8_t* attn_ws = nullptr;
   size_t attn_ws_bytes = 0;
   // FP16 decode rows: the o_proj runs inside the attention's workgroup merge
@@ -528,7 +534,7 @@ int llm_decoder::layer_attn(int l, hipStream_t st, const Rows& R, PaPlan* plan) 
   RET_IF(kv_cache_view(kv, l, &view));
   view.page_table += (size_t)R.table_row0 * H * view.max_tiles;  // rows r0..
   view.num_beams -= R.table_row0;
-  if (R.prefill_row >= 0 && pa_prefill_supported(&view) && !plan) {
+  if (R.prefill_row >= 0 && !R.mixed && pa_prefill_supported(&view) && !plan) {
     // one MFMA pass over the chunk (K/V pages read once per 32 queries), then
     // the o_proj input conversion the decode merge would have fused
     PaRowOutputs ro;
@@ -801,6 +807,31 @@ int llm_decoder::oproj_range_status() {
   return report_range(f);
 }
 
+// Buffers for one layer pass of C prompt tokens.
+int llm_decoder::ensure_prefill(int C) {
+  if (C <= pf_cap) return LLM_OK;
+  const size_t C16 = ((size_t)C + 15) / 16 * 16;
+  RET_IF(px.alloc((size_t)C * hid));
+  RET_IF(pq.alloc((size_t)C * hid));
+  RET_IF(po.alloc((size_t)C * hid));
+  RET_IF(ph1.alloc((size_t)C * inter));
+  RET_IF(psa.alloc((size_t)C));
+  RET_IF(pact.alloc(C16 * std::max(hid, inter) * (wdtype == LLM_I8 ? 1 : 4)));  // F16: act, act2
+  RET_IF(pmeta.alloc((size_t)4 * C));
+  pws_bytes = 16;
+  for (int b = 1; b <= C; ++b)
+    pws_bytes = std::max(pws_bytes, pa_decode_workspace_bytes(b, H, D, max_tiles, 0));
+  {  // the MFMA prefill's split partials (its split count is bounded at any p0)
+    pa_kv_view v0;
+    RET_IF(kv_cache_view(kv, 0, &v0));
+    for (int b = 1; b <= C; ++b)
+      pws_bytes = std::max(pws_bytes, pa_prefill_ws_bytes(&v0, cfg.max_seq_len - b, b));
+  }
+  RET_IF(pws.alloc(pws_bytes));
+  pf_cap = C;
+  return LLM_OK;
+}
+
 // Chunked prefill of `n` prompt tokens of active row `row` (the reference's
 // is_prefill pass, attention/attention_cuda.hpp:21): the chunk's tokens are
 // the rows of one layer pass — M = chunk-size weight GEMMs, the K/V of every
@@ -816,27 +847,7 @@ int llm_decoder::prefill(int row, const int32_t* toks, int n, hipStream_t st) {
   LLM_REQUIRE(h_pos[row] + n < cfg.max_seq_len, "prefill: prompt exceeds max_seq_len");
   for (int i = 0; i < n; ++i) LLM_REQUIRE(toks[i] >= 0 && toks[i] < V, "prefill: token id out of range");
   const int C = std::min(n, kPrefillChunk);
-  if (C > pf_cap) {
-    const size_t C16 = ((size_t)C + 15) / 16 * 16;
-    RET_IF(px.alloc((size_t)C * hid));
-    RET_IF(pq.alloc((size_t)C * hid));
-    RET_IF(po.alloc((size_t)C * hid));
-    RET_IF(ph1.alloc((size_t)C * inter));
-    RET_IF(psa.alloc((size_t)C));
-    RET_IF(pact.alloc(C16 * std::max(hid, inter) * (wdtype == LLM_I8 ? 1 : 4)));  // F16: act, act2
-    RET_IF(pmeta.alloc((size_t)4 * C));
-    pws_bytes = 16;
-    for (int b = 1; b <= C; ++b)
-      pws_bytes = std::max(pws_bytes, pa_decode_workspace_bytes(b, H, D, max_tiles, 0));
-    {  // the MFMA prefill's split partials (its split count is bounded at any p0)
-      pa_kv_view v0;
-      RET_IF(kv_cache_view(kv, 0, &v0));
-      for (int b = 1; b <= C; ++b)
-        pws_bytes = std::max(pws_bytes, pa_prefill_ws_bytes(&v0, cfg.max_seq_len - b, b));
-    }
-    RET_IF(pws.alloc(pws_bytes));
-    pf_cap = C;
-  }
+  RET_IF(ensure_prefill(C));
   KvCache* k = kv_impl(kv);
   std::vector<int32_t> meta((size_t)4 * C), pc(2);
   for (int c0 = 0; c0 < n; c0 += C) {
@@ -881,6 +892,74 @@ int llm_decoder::prefill(int row, const int32_t* toks, int n, hipStream_t st) {
     }
     LLM_HIP_RET(hipStreamSynchronize(st));  // meta / pc staging reused next chunk
   }
+  return LLM_OK;
+}
+
+// The serving engine's step: the new tokens of several sequences as the rows
+// of one layer pass (one sequence: the prefill form), logits of the wanted
+// rows into logits_dev.  Positions and page-table rows come with the entries;
+// the fixed-batch state of the step graph (h_pos, tokens) is not used.
+int llm_decoder::forward_mixed(const std::vector<StepSeq>& seqs, float* logits_dev,
+                               hipStream_t st) {
+  LLM_REQUIRE(weights_ready, "decoder: weights not loaded");
+  int n = 0;
+  for (const StepSeq& s : seqs) {
+    LLM_REQUIRE(s.slot >= 0 && s.slot < maxB && s.n >= 1 && s.p0 >= 0 &&
+                    s.p0 + s.n <= cfg.max_seq_len,
+                "decoder: a sequence grows past max_seq_len");
+    n += s.n;
+  }
+  LLM_REQUIRE(n >= 1 && n <= kPrefillChunk, "decoder: too many tokens in one step");
+  RET_IF(ensure_prefill(kPrefillChunk));
+  const int C = pf_cap;
+  KvCache* k = kv_impl(kv);
+  {
+    std::lock_guard<std::mutex> gk(k->mu);
+    for (const StepSeq& s : seqs)
+      for (int t = s.p0; t < s.p0 + s.n; t = (t / TS + 1) * TS) RET_IF(k->prepare_append(s.slot, t));
+    RET_IF(k->sync(st));
+  }
+  std::vector<int32_t> m((size_t)4 * C);
+  std::vector<int> want;
+  int i = 0;
+  for (const StepSeq& s : seqs) {
+    for (int w = 0; w < s.n_want; ++w) want.push_back(i + s.want[w]);
+    for (int j = 0; j < s.n; ++j, ++i) {
+      LLM_REQUIRE(s.tokens[j] >= 0 && s.tokens[j] < V, "decoder: token id out of range");
+      m[i] = s.p0 + j;
+      m[C + i] = s.p0 + j + 1;
+      m[2 * C + i] = s.slot;
+      m[3 * C + i] = s.tokens[j];
+    }
+  }
+  LLM_HIP_RET(hipMemcpyAsync(pmeta.p, m.data(), m.size() * sizeof(int32_t), hipMemcpyHostToDevice, st));
+  Rows R;
+  R.n = n;
+  R.x = px.p; R.q = pq.p; R.o = po.p; R.h1 = ph1.p; R.act = pact.p; R.sa = psa.p;
+  if (wdtype == LLM_F16)
+    R.act2 = pact.p + (((size_t)C + 15) / 16 * 16) * std::max(hid, inter) * 2;
+  R.pos = pmeta.p; R.ctx = pmeta.p + C; R.beam_rows = pmeta.p + 2 * C;
+  R.mixed = seqs.size() > 1;
+  R.prefill_row = seqs[0].slot;
+  R.prefill_p0 = seqs[0].p0;
+  R.attn_ws = pws.p; R.attn_ws_bytes = pws_bytes;
+  LLM_HIP_RET(launch_embed(emb.p, pmeta.p + 3 * C, n, hid, V, px.p, st));
+  embed_src = LnSource{};
+  for (int l = 0; l < L; ++l) {
+    RET_IF(layer_pre(l, st, R));
+    RET_IF(layer_attn(l, st, R));
+    RET_IF(layer_post(l, st, R));
+  }
+  // the wanted rows together (in the attention output's buffer), then the LM head
+  for (size_t w0 = 0, w1; w0 < want.size(); w0 = w1) {
+    for (w1 = w0 + 1; w1 < want.size() && want[w1] == want[w1 - 1] + 1; ++w1) {}
+    LLM_HIP_RET(hipMemcpyAsync(po.p + w0 * hid, px.p + (size_t)want[w0] * hid,
+                               sizeof(float) * (w1 - w0) * hid, hipMemcpyDeviceToDevice, st));
+  }
+  if (!want.empty())
+    LLM_HIP_RET(launch_lm_head(po.p, emb_packed.p, logits_dev, (int)want.size(), V, hid, nullptr,
+                               nullptr, st));
+  LLM_HIP_RET(hipStreamSynchronize(st));  // m is on this stack
   return LLM_OK;
 }
 
@@ -1379,3 +1458,69 @@ extern "C" int llm_decoder_load_quantized_weights(llm_decoder* d, const char* di
                      q2.data(), s2.data(), b2.data()};
   return llm_decoder_set_int8_weights(d, &w);
 }
+
+// ---------------------------------------------------------------------------
+// the decoders in the model registry (csrc/model.hpp)
+// ---------------------------------------------------------------------------
+namespace {
+
+class DecoderModel final : public StepModel {
+ public:
+  ~DecoderModel() override { llm_decoder_destroy(d_); }
+  int init(const Json& c, const std::string& dir, const ModelOptions& o, int wdtype) {
+    if (o.dtype == LLM_F32)
+      return fail(LLM_ERR_UNSUPPORTED, "model: " + c["architecture"].str +
+                                           " runs in its own precision, not float32");
+    llm_decoder_config g{};
+    g.num_layers = (int)c["num_layers"].num;
+    g.num_heads = (int)c["num_heads"].num;
+    g.head_dim = (int)c["head_dim"].num;
+    g.hidden_dim = c.has("hidden_dim") ? (int)c["hidden_dim"].num : g.num_heads * g.head_dim;
+    g.vocab_size = (int)c["vocab_size"].num;
+    g.inter_dim = (int)c["inter_dim"].num;
+    g.page_size = c.has("page_size") ? (int)c["page_size"].num : 16;
+    g.attn_scale = c.has("attn_scale") ? (float)c["attn_scale"].num : 1.f;
+    g.weight_dtype = wdtype;
+    g.max_batch = o.max_seqs;
+    LLM_REQUIRE(g.page_size > 0, "config.json: page_size");
+    pages_ = (o.max_tokens + g.page_size - 1) / g.page_size;
+    long long len = o.max_seq_len > 0 ? o.max_seq_len : pages_ * g.page_size;
+    if (c.has("max_seq_len")) len = std::min(len, (long long)c["max_seq_len"].num);
+    g.max_seq_len = (int)std::min<long long>(len, 1 << 28);
+    g.num_pages = pages_ * g.num_layers * g.num_heads;
+    RET_IF(llm_decoder_create(&g, &d_));
+    const bool quantised = wdtype == LLM_I8 && std::ifstream(dir + "/embedding.f16").good();
+    return quantised ? llm_decoder_load_quantized_weights(d_, dir.c_str())
+                     : llm_decoder_load_weights(d_, dir.c_str());
+  }
+  int vocab() const override { return d_->V; }
+  int max_seq_len() const override { return d_->cfg.max_seq_len; }
+  int max_step_tokens() const override { return llm_decoder::kPrefillChunk; }
+  int page_tokens() const override { return d_->TS; }
+  long long pool_tokens() const override { return pages_ * d_->TS; }
+  long long free_tokens() const override {
+    return kv_cache_free_pages(d_->kv) / ((long long)d_->L * d_->H) * d_->TS;
+  }
+  int forward(const std::vector<StepSeq>& batch, float* logits, hipStream_t st) override {
+    std::lock_guard<std::mutex> g(d_->mu);
+    return d_->forward_mixed(batch, logits, st);
+  }
+  int release(int slot) override { return kv_cache_release(d_->kv, slot); }
+
+ private:
+  llm_decoder* d_ = nullptr;
+  long long pages_ = 0;
+};
+
+template <int WDTYPE>
+int make_decoder(const Json& c, const std::string& dir, const ModelOptions& o,
+                 std::unique_ptr<StepModel>* out) {
+  auto m = std::make_unique<DecoderModel>();
+  RET_IF(m->init(c, dir, o, WDTYPE));
+  *out = std::move(m);
+  return LLM_OK;
+}
+const ModelRegistrar reg_f16("CUDADecoder", &make_decoder<LLM_F16>);
+const ModelRegistrar reg_i8("INT8Decoder", &make_decoder<LLM_I8>);
+
+}  // namespace

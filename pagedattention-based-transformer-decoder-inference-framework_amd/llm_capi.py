@@ -45,6 +45,21 @@ class PaDecodeOptions(ctypes.Structure):
                 ("scores_out", c_void_p)]
 
 
+class EngineConfig(ctypes.Structure):
+    _fields_ = [("dtype", c_int), ("max_seqs", c_int), ("max_tokens", c_ll),
+                ("max_seq_len", c_int), ("max_step_tokens", c_int)]
+
+
+class EngineEntry(ctypes.Structure):
+    _fields_ = [("seq", c_int), ("tokens", c_void_p), ("n", c_int), ("want", c_void_p),
+                ("n_want", c_int)]
+
+
+class RequestParams(ctypes.Structure):
+    _fields_ = [("max_new_tokens", c_int), ("temperature", c_float), ("top_k", c_int),
+                ("top_p", c_float), ("seed", ctypes.c_uint64), ("eos_token", c_int)]
+
+
 class LlmError(RuntimeError):
     def __init__(self, status: int, msg: str):
         super().__init__(f"[llm status {status}] {msg}")
@@ -121,6 +136,24 @@ _SIGS = {
     "kv_tiles_inspect": (c_int, [ctypes.c_char_p, ctypes.c_longlong, ctypes.POINTER(c_int)]),
     "llm_decoder_oproj_status": (c_int, [c_void_p, ctypes.POINTER(c_int),
                                          ctypes.POINTER(ctypes.c_longlong)]),
+    "llm_model_architectures": (ctypes.c_char_p, []),
+    "llm_engine_create": (c_int, [ctypes.c_char_p, ctypes.POINTER(EngineConfig),
+                                  ctypes.POINTER(c_void_p)]),
+    "llm_engine_destroy": (None, [c_void_p]),
+    "llm_engine_vocab": (c_int, [c_void_p]),
+    "llm_engine_max_seq_len": (c_int, [c_void_p]),
+    "llm_engine_page_tokens": (c_int, [c_void_p]),
+    "llm_engine_free_tokens": (c_ll, [c_void_p]),
+    "llm_engine_open": (c_int, [c_void_p, c_i32p]),
+    "llm_engine_close": (c_int, [c_void_p, c_int]),
+    "llm_engine_seq_len": (c_int, [c_void_p, c_int]),
+    "llm_engine_step": (c_int, [c_void_p, ctypes.POINTER(EngineEntry), c_int, c_void_p]),
+    "llm_engine_set_tap": (c_int, [c_void_p, c_void_p]),
+    "llm_engine_layer_runs": (c_int, [c_void_p]),
+    "llm_engine_width": (c_int, [c_void_p]),
+    "llm_engine_submit": (c_int, [c_void_p, c_void_p, c_int, ctypes.POINTER(RequestParams), c_i32p]),
+    "llm_engine_run": (c_int, [c_void_p, c_i32p]),
+    "llm_engine_result": (c_int, [c_void_p, c_int, c_void_p, c_int, c_i32p, c_i32p]),
 }
 
 _lib = None
