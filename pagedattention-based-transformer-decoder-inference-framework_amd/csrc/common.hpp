@@ -115,6 +115,16 @@ __device__ __forceinline__ float wave_max(float x) {
   return x;
 }
 
+// wave_max through DPP moves inside the 16-lane rows
+__device__ __forceinline__ float wave_max_dpp(float x) {
+  x = fmaxf(x, mov_dpp<0xB1>(x));
+  x = fmaxf(x, mov_dpp<0x4E>(x));
+  x = fmaxf(x, mov_dpp<0x141>(x));
+  x = fmaxf(x, mov_dpp<0x140>(x));
+  x = fmaxf(x, __shfl_xor(x, 16, 64));
+  return fmaxf(x, __shfl_xor(x, 32, 64));
+}
+
 __device__ __forceinline__ float wave_sum(float x) {
 #pragma unroll
   for (int off = 32; off >= 1; off >>= 1) x += __shfl_xor(x, off, 64);
@@ -126,6 +136,18 @@ __device__ __forceinline__ int wave_id_uniform() {
 }
 
 __device__ __forceinline__ int lane_id() { return threadIdx.x & 63; }
+
+// 16 bytes per lane from memory straight into LDS, lane l's at lds + 16 l (lds:
+// the same for the whole wave).  Written as assembly so the compiler does not
+// order later LDS reads behind it: a wave calls wait_lds_loads() and then the
+// workgroup barrier before anyone reads what was loaded.
+__device__ __forceinline__ void load_to_lds(const void* src, void* lds) {
+  const uint32_t at = __builtin_amdgcn_readfirstlane(
+      (uint32_t)(uintptr_t)(__attribute__((address_space(3))) void*)lds);
+  asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(at), "v"(src)
+               : "memory", "m0");
+}
+__device__ __forceinline__ void wait_lds_loads() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
 
 // Offset of activation element (m, k) in MFMA A-fragment order ("packed A"):
 // one contiguous 1 KiB block per (16-row tile, k-step), lane l of the block

@@ -58,8 +58,9 @@ namespace {
 
 constexpr int kDefaultStepTokens = 2048;
 constexpr int kMaxSplits = 64;
-constexpr int kTargetGroups = 768;   // workgroups an attention launch is split up to
+constexpr int kTargetGroups = 512;   // workgroups an attention launch is split up to: 2 per CU
 constexpr int kMinSplitPages = 4;    // a page per wave
+constexpr size_t kMaxGraphs = 256;   // decode shapes kept captured
 constexpr size_t kKeepBytes = (size_t)192 << 20;  // weights up to this stay in the Infinity Cache
 
 int check_config(const LayerStackConfig& c, const ModelOptions& o) {
@@ -477,9 +478,9 @@ int LayerStack::ensure_rows(int M) {
   return LLM_OK;
 }
 
-// The row tiles of one attention launch: sequences that bring at most 16 rows
-// per key/value head (big false) or more, split over their pages until the
-// launch holds about kTargetGroups workgroups.
+// The row tiles of one attention launch: sequences that bring few rows per
+// key/value head (big false) or many, split over their pages until the launch
+// holds about kTargetGroups workgroups; long tiles first.
 void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
                      std::vector<GqaItem>& items, std::vector<GqaMerge>& merges, Launch& l) {
   l = Launch();
@@ -488,7 +489,7 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
   int max_pages = 1, tok0 = 0;
   for (const StepSeq& s : batch) {
     const int rows = s.n * p.R;
-    if ((rows > 16) != big) continue;
+    if ((rows > kGqaSmallRows) != big) continue;
     tiles += (rows + l.tile_rows - 1) / l.tile_rows;
     max_pages = std::max(max_pages, (s.p0 + s.n - 1) / kPageTokens + 1);
   }
@@ -501,7 +502,7 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
     const int rows = s.n * p.R;
     const int t0 = tok0;
     tok0 += s.n;
-    if ((rows > 16) != big) continue;
+    if ((rows > kGqaSmallRows) != big) continue;
     for (int r0 = 0; r0 < rows; r0 += l.tile_rows) {
       const int last = s.p0 + (std::min(r0 + l.tile_rows, rows) - 1) / p.R;
       const int pages = last / kPageTokens + 1;
@@ -517,6 +518,10 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
       }
     }
   }
+  if (big)
+    std::stable_sort(items.begin(), items.end(), [](const GqaItem& x, const GqaItem& y) {
+      return x.page1 - x.page0 > y.page1 - y.page0;
+    });
 }
 
 int LayerStack::build_meta(const std::vector<StepSeq>& batch, int M, int n_want, hipStream_t st) {
@@ -824,6 +829,10 @@ int LayerStack::forward(const std::vector<StepSeq>& batch, float* logits, hipStr
       key.insert(key.end(), {l->n_items, l->n_merges});
   auto it = graphs_.find(key);
   if (it == graphs_.end()) {  // first of its shape: run it, capture the next
+    if (graphs_.size() >= kMaxGraphs) {  // shapes of contexts long gone
+      LLM_HIP_RET(hipStreamSynchronize(st));
+      clear_graphs();
+    }
     graphs_[key] = nullptr;
     return enqueue(M, n_want, logits, st);
   }

@@ -79,7 +79,7 @@ struct MmGrouped {
   const float* weight = nullptr;    // [M * top], by token * top + choice
   int n_routed = 0, top = 0, M = 0;
   int max_tiles = 0;                // grid bound
-  int tile_rows = 16;               // 16 or 64: rows of a tile list entry
+  int tile_rows = 16;               // 16, 64 or 128: rows of a tile list entry
   int max_n = 0;                    // widest group's columns
   int min_ks = 0;
   const void* h = nullptr;          // [M][ldh] tokens' rows

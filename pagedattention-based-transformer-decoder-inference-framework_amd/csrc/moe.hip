@@ -10,16 +10,17 @@
 namespace llm {
 namespace {
 
-constexpr int kLaneExperts = kMaxExperts / 64;
 constexpr int kSortThreads = 1024;
-constexpr int kFusedTokens = 128;
+constexpr int kFusedTokens = 16;  // a token per wave of the one workgroup
+constexpr int kFusedTop = 32;
 
-// One wave: token m's choices.  Lane l holds experts l, l + 64, ...
-__device__ __forceinline__ void choose(const RouteArgs& a, int m) {
+// One wave: token m's choices.  Lane l holds LE experts: l, l + 64, ...
+template <int LE>
+__device__ __forceinline__ void choose(const RouteArgs& a, int m, int32_t* choice) {
   const int lane = lane_id();
-  float s[kLaneExperts], key[kLaneExperts];
+  float s[LE], key[LE];
 #pragma unroll
-  for (int j = 0; j < kLaneExperts; ++j) {
+  for (int j = 0; j < LE; ++j) {
     const int e = lane + 64 * j;
     s[j] = 0.f;
     key[j] = -INFINITY;
@@ -29,36 +30,41 @@ __device__ __forceinline__ void choose(const RouteArgs& a, int m) {
     }
   }
   for (int k = 0; k < a.top; ++k) {
-    float best = -INFINITY, bs = 0.f;
-    int be = 0x7fffffff;
+    float best = key[0];
 #pragma unroll
-    for (int j = 0; j < kLaneExperts; ++j)
-      if (key[j] > best) { best = key[j]; be = lane + 64 * j; bs = s[j]; }
+    for (int j = 1; j < LE; ++j) best = fmaxf(best, key[j]);
+    best = wave_max_dpp(best);
+    // the lowest expert that has it (scores that are not numbers match nothing:
+    // any valid expert then)
+    int be = k;
+    float bs = 0.f;
 #pragma unroll
-    for (int off = 32; off >= 1; off >>= 1) {
-      const float ov = __shfl_xor(best, off, 64), os = __shfl_xor(bs, off, 64);
-      const int oe = __shfl_xor(be, off, 64);
-      if (ov > best || (ov == best && oe < be)) { best = ov; be = oe; bs = os; }
+    for (int j = LE - 1; j >= 0; --j) {
+      const unsigned long long hit = __ballot(key[j] == best);
+      if (hit) {
+        const int l = __ffsll(hit) - 1;
+        be = l + 64 * j;
+        bs = __shfl(s[j], l, 64);
+      }
     }
-    // (scores that are not numbers choose nothing; any valid expert then)
     if (be >= a.experts) be = k;
     if (lane == 0) {
-      a.choice[(size_t)m * a.top + k] = be;
+      choice[(size_t)m * a.top + k] = be;
       a.weight[(size_t)m * a.top + k] = bs * a.scale;
     }
 #pragma unroll
-    for (int j = 0; j < kLaneExperts; ++j)
+    for (int j = 0; j < LE; ++j)
       if (be == lane + 64 * j) key[j] = -INFINITY;
   }
 }
 
 // One workgroup: counts per expert, their starts, the tile list, the order.
-__device__ __forceinline__ void sort_assignments(const RouteArgs& a, int* cnt, int* start,
-                                                 int* tile0) {
+__device__ __forceinline__ void sort_assignments(const RouteArgs& a, const int32_t* choice, int* cnt,
+                                                 int* start, int* tile0) {
   const int n = a.M * a.top, E = a.experts;
   for (int e = threadIdx.x; e < E; e += kSortThreads) cnt[e] = 0;
   __syncthreads();
-  for (int i = threadIdx.x; i < n; i += kSortThreads) atomicAdd(&cnt[a.choice[i]], 1);
+  for (int i = threadIdx.x; i < n; i += kSortThreads) atomicAdd(&cnt[choice[i]], 1);
   __syncthreads();
   if (threadIdx.x < 64) {  // exclusive sums of rows and tiles, 64 experts at a time
     int rows = 0, tiles = 0;
@@ -95,27 +101,30 @@ __device__ __forceinline__ void sort_assignments(const RouteArgs& a, int* cnt, i
   for (int e = threadIdx.x; e < E; e += kSortThreads) cnt[e] = start[e];
   __syncthreads();
   for (int i = threadIdx.x; i < n; i += kSortThreads) {
-    const int at = atomicAdd(&cnt[a.choice[i]], 1);
+    const int at = atomicAdd(&cnt[choice[i]], 1);
     a.perm[at] = i;
   }
 }
 
+template <int LE>
 __global__ __launch_bounds__(kSortThreads) void route_small_kernel(RouteArgs a) {
   __shared__ int cnt[kMaxExperts], start[kMaxExperts], tile0[kMaxExperts + 1];
-  for (int m = wave_id_uniform(); m < a.M; m += kSortThreads / 64) choose(a, m);
-  __syncthreads();  // (the choices go through the workgroup's own CU cache)
-  __threadfence_block();
-  sort_assignments(a, cnt, start, tile0);
+  __shared__ int32_t choice[kFusedTokens * kFusedTop];
+  const int m = wave_id_uniform();
+  if (m < a.M) choose<LE>(a, m, choice);
+  __syncthreads();
+  sort_assignments(a, choice, cnt, start, tile0);
 }
 
+template <int LE>
 __global__ __launch_bounds__(256) void route_choose_kernel(RouteArgs a) {
   const int m = blockIdx.x * 4 + wave_id_uniform();
-  if (m < a.M) choose(a, m);
+  if (m < a.M) choose<LE>(a, m, a.choice);
 }
 
 __global__ __launch_bounds__(kSortThreads) void route_sort_kernel(RouteArgs a) {
   __shared__ int cnt[kMaxExperts], start[kMaxExperts], tile0[kMaxExperts + 1];
-  sort_assignments(a, cnt, start, tile0);
+  sort_assignments(a, a.choice, cnt, start, tile0);
 }
 
 }  // namespace
@@ -127,16 +136,23 @@ int route_max_tiles(int M, int top, int experts, bool shared, int tile_rows) {
   return routed + (shared ? (M + tile_rows - 1) / tile_rows : 0);
 }
 
-hipError_t route(const RouteArgs& a, hipStream_t st) {
-  if (a.M <= 0) return hipSuccess;
-  if (a.M <= kFusedTokens) {
-    hipLaunchKernelGGL(route_small_kernel, dim3(1), dim3(kSortThreads), 0, st, a);
+template <int LE>
+static hipError_t route_le(const RouteArgs& a, hipStream_t st) {
+  if (a.M <= kFusedTokens && a.top <= kFusedTop) {
+    hipLaunchKernelGGL(route_small_kernel<LE>, dim3(1), dim3(kSortThreads), 0, st, a);
     return hipGetLastError();
   }
-  hipLaunchKernelGGL(route_choose_kernel, dim3((a.M + 3) / 4), dim3(256), 0, st, a);
+  hipLaunchKernelGGL(route_choose_kernel<LE>, dim3((a.M + 3) / 4), dim3(256), 0, st, a);
   if (hipError_t e = hipGetLastError()) return e;
   hipLaunchKernelGGL(route_sort_kernel, dim3(1), dim3(kSortThreads), 0, st, a);
   return hipGetLastError();
+}
+
+hipError_t route(const RouteArgs& a, hipStream_t st) {
+  if (a.M <= 0) return hipSuccess;
+  if (a.experts <= 64) return route_le<1>(a, st);
+  if (a.experts <= 128) return route_le<2>(a, st);
+  return a.experts <= 256 ? route_le<4>(a, st) : route_le<kMaxExperts / 64>(a, st);
 }
 
 }  // namespace llm

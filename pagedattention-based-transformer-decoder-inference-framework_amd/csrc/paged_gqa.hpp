@@ -48,6 +48,7 @@ struct GqaArgs {
   float* part_ml = nullptr;  // [part][G][tile_rows][2]
 };
 constexpr int kGqaMaxDim = 256;
+constexpr int kGqaSmallRows = 64;  // sequences up to this many rows take tiles of 16
 // Rows per tile for sequences that bring `rows` rows per key/value head.
 int gqa_tile_rows(int dtype, int Dp, int Dvp, int rows);
 inline int gqa_part_dim(int Dv) { return (Dv + 15) / 16 * 16; }

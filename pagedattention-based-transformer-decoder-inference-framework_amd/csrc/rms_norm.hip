@@ -47,6 +47,15 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
     if (c < nv) x[j] = a.embed == 1 ? embed_at(c) : *reinterpret_cast<const f32x4*>(xr + 4 * c);
   }
   const float inv_w = 1.f / (float)a.width;
+  // the norm weights fly while the rows are summed
+  f32x4 wpost[NV], wpre[NV];
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    const int c = threadIdx.x + j * THREADS;
+    wpost[j] = wpre[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (c < nv && a.w_post) wpost[j] = *reinterpret_cast<const f32x4*>(a.w_post + 4 * c);
+    if (c < nv && a.w_pre) wpre[j] = *reinterpret_cast<const f32x4*>(a.w_pre + 4 * c);
+  }
   if (a.w_post) {
     f32x4 y[NV];
     float ss = 0.f;
@@ -55,10 +64,18 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
       const int c = threadIdx.x + j * THREADS;
       f32x4 s = {0.f, 0.f, 0.f, 0.f};
       if (c < nv) {
-        for (int q = 0; q < a.parts; ++q)
-          s += *reinterpret_cast<const f32x4*>(a.y + ((size_t)m * a.parts + q) * a.ldy + 4 * c);
+        const float* y0 = a.y + (size_t)m * a.parts * a.ldy + 4 * c;
         if (a.shared)
-          s += *reinterpret_cast<const f32x4*>(a.y + ((size_t)a.M_y * a.parts + m) * a.ldy + 4 * c);
+          s = *reinterpret_cast<const f32x4*>(a.y + ((size_t)a.M_y * a.parts + m) * a.ldy + 4 * c);
+        for (int q = 0; q < a.parts; q += 4) {  // four parts' loads in flight
+          f32x4 v[4];
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            v[u] = *reinterpret_cast<const f32x4*>(y0 + (size_t)min(q + u, a.parts - 1) * a.ldy);
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+            if (q + u < a.parts) s += v[u];
+        }
 #pragma unroll
         for (int e = 0; e < 4; ++e)
           if (4 * c + e >= a.width) s[e] = 0.f;
@@ -70,7 +87,7 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int c = threadIdx.x + j * THREADS;
-      if (c < nv) x[j] += y[j] * r * *reinterpret_cast<const f32x4*>(a.w_post + 4 * c);
+      if (c < nv) x[j] += y[j] * r * wpost[j];
     }
   }
   if (a.embed == 2) {
@@ -97,7 +114,7 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
   for (int j = 0; j < NV; ++j) {
     const int c = threadIdx.x + j * THREADS;
     if (c >= nv) continue;
-    const f32x4 o = x[j] * r * *reinterpret_cast<const f32x4*>(a.w_pre + 4 * c);
+    const f32x4 o = x[j] * r * wpre[j];
     if constexpr (sizeof(T) == 2)
       *reinterpret_cast<bf16x4*>(hr + 4 * c) =
           bf16x4{(__bf16)o[0], (__bf16)o[1], (__bf16)o[2], (__bf16)o[3]};

@@ -268,19 +268,28 @@ static int row_vpt(int cols) {
 }
 
 // Argmax per row, first maximum wins (std::max_element).
-__global__ __launch_bounds__(kRowThreads) void argmax_kernel(const float* __restrict__ logits,
-                                                             int V, int32_t* __restrict__ out,
-                                                             int32_t* __restrict__ out2,
-                                                             int out2_stride) {
-  __shared__ float shv[kRowThreads];
-  __shared__ int shi[kRowThreads];
+constexpr int kArgmaxThreads = 1024;
+__global__ __launch_bounds__(kArgmaxThreads) void argmax_kernel(const float* __restrict__ logits,
+                                                                int V, int32_t* __restrict__ out,
+                                                                int32_t* __restrict__ out2,
+                                                                int out2_stride) {
+  __shared__ float shv[kArgmaxThreads];
+  __shared__ int shi[kArgmaxThreads];
   const int r = blockIdx.x;
   const float* l = logits + (size_t)r * V;
   float best = -INFINITY;
   int bi = 0x7fffffff;
-  for (int i = threadIdx.x; i < V; i += blockDim.x) {
-    const float v = l[i];
-    if (v > best) { best = v; bi = i; }  // strided scan: first index per thread
+  constexpr int U = 8;  // loads in flight
+  for (int i0 = threadIdx.x; i0 < V; i0 += U * kArgmaxThreads) {
+    float v[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int i = i0 + u * kArgmaxThreads;
+      v[u] = i < V ? l[i] : -INFINITY;
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)  // strided scan: first index per thread
+      if (v[u] > best) { best = v[u]; bi = i0 + u * kArgmaxThreads; }
   }
   shv[threadIdx.x] = best;
   shi[threadIdx.x] = bi;
@@ -438,7 +447,7 @@ hipError_t launch_advance(int32_t* pos, int32_t* ctx, int n, hipStream_t st) {
 
 hipError_t launch_argmax(const float* logits, int rows, int V, int32_t* out, int32_t* out2,
                          int out2_stride, hipStream_t st) {
-  hipLaunchKernelGGL(argmax_kernel, dim3(rows), dim3(kRowThreads), 0, st, logits, V, out, out2,
+  hipLaunchKernelGGL(argmax_kernel, dim3(rows), dim3(kArgmaxThreads), 0, st, logits, V, out, out2,
                      out2_stride);
   return hipGetLastError();
 }

@@ -267,11 +267,11 @@ def test_batch_alone_and_step_size_give_the_same(serve):
 
 
 # --------------------------------------------------------- keys that stand out
-def needle_model(seed):
+def needle_model(seed, heads=4):
     """A model whose token 1 looks for token 0 wherever it is: its query meets
     that key, in dimensions that are not rotated, far above every other score,
     and token 0's value is unlike the others'."""
-    a = T.attn(heads=4, kv_heads=2, dim=32, vdim=16, rot=8)
+    a = T.attn(heads=heads, kv_heads=2, dim=32, vdim=16, rot=8)
     cfg = T.config([(a, None)], width=64, vocab=60)
     w = T.weights(cfg, seed)
     W = cfg["width"]
@@ -286,10 +286,10 @@ def needle_model(seed):
     for h in range(2):
         w["l0.mix.k"][32 * h + 20, 0] = 4.0      # key of token 0
         w["l0.mix.v"][16 * h:16 * h + 16, 0] = np.linspace(-1, 1, 16)
-    for h in range(4):
+    for h in range(heads):
         w["l0.mix.q"][32 * h + 20, 1] = 4.0      # query of token 1: score 16 * 64 / sqrt(32)
+        w["l0.mix.q"][32 * h + 20, 2:] = 0
     w["l0.mix.k"][[20, 52], 1:] = 0
-    w["l0.mix.q"][[20, 52, 84, 116], 2:] = 0
     return cfg, {k: T.to_bf16(v) for k, v in w.items()}
 
 
@@ -321,6 +321,29 @@ def test_one_key_at_page_borders_and_far_away(serve, dtype, decoded):
         assert e.max() < (T.FP32_TOL if dtype == "float32" else T.BF16_TOL), (at, e)
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("group", [2, 8])
+def test_far_keys_in_long_contexts(serve, dtype, group):
+    """Contexts long enough that every launch form splits the keys: whole
+    prompts, prompts past the step size, short portions and single tokens far
+    from the key; a heavy sink that counts once whatever the splits."""
+    cfg, w = needle_model(33, heads=2 * group)
+    w["l0.mix.sink"] = T.to_bf16(np.linspace(8, 11, 2 * group))
+    n = 1200
+    base = 2 + np.random.default_rng(34).integers(0, cfg["vocab"] - 2, n).astype(np.int32)
+    eng = serve(cfg, w, dtype, max_tokens=2 * 1536, max_seqs=2, max_step_tokens=700)
+    for at, asked in ((3, [700, 1199]), (1023, [1024, 1190])):
+        t = base.copy()
+        t[at], t[asked] = 0, 1
+        want = T.logits(cfg, w, t)[asked]
+        gone = np.where(np.arange(n) == at, base, t)
+        assert T.row_error(T.logits(cfg, w, gone)[asked], want).min() > 0.3
+        for steps in ([[(0, n)]],
+                      [[(0, 400)], [(0, 300)], [(0, 3)], [(0, 460)]] + [[(0, 2)]] * 10 + [[(0, 1)]] * 17):
+            got = T.replay(eng, {0: t}, steps)[0][asked]
+            T.check_rows(got, want, dtype)
+
+
 def test_key_just_ahead_is_not_seen(serve):
     """The standing-out key one place after the query, in one portion and across
     the portion's edge."""
@@ -330,7 +353,8 @@ def test_key_just_ahead_is_not_seen(serve):
         t = 2 + np.random.default_rng(p).integers(0, cfg["vocab"] - 2, 140).astype(np.int32)
         t[p], t[p + 1] = 1, 0
         want = T.logits(cfg, w, t)
-        for steps in ([[(0, 140)]], [[(0, p + 1)], [(0, 139 - p)]], [[(0, p)]] + [[(0, 1)]] * 5):
+        for steps in ([[(0, 140)]], [[(0, p + 1)], [(0, 139 - p)]], [[(0, p)]] + [[(0, 1)]] * 5,
+                      [[(0, 140 - 2)], [(0, 2)]]):
             got = T.replay(eng, {0: t}, steps)[0]
             T.check_rows(got, want[:len(got)], "float32")
 
