@@ -57,8 +57,8 @@ struct LayerStackConfig {
   int vocab = 0, width = 0;
   float eps = 1e-5f;
   std::vector<LayerSpec> layers;
-  // layers [loop_start, loop_stop) run loop_times times in a row; each pass but
-  // the first adds the embedding output to the residual before its first layer
+  // layers [loop_start, loop_stop) are passed through loop_times times; a repeated
+  // pass starts with the tokens' embeddings added to the residual once more
   int loop_start = 0, loop_stop = 0, loop_times = 1;
 };
 

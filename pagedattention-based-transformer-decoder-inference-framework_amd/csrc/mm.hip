@@ -469,7 +469,7 @@ hipError_t launch(const KernelArgs& p, hipStream_t st) {
                               : stream<T, EPI, 1, 2>(p, b16, N, st);
   // prompt rows: blocks once there are enough of them, else 32-row streams
   const int n128 = (N + 127) / 128;
-  if ((M + 127) / 128 * n128 >= 160) return blocks<T, EPI, 8, 2>(p, (M + 127) / 128, N, st);
+  if ((M + 127) / 128 * n128 >= 256) return blocks<T, EPI, 8, 2>(p, (M + 127) / 128, N, st);
   if ((M + 63) / 64 * n128 >= 128) return blocks<T, EPI, 4, 1>(p, (M + 63) / 64, N, st);
   return stream<T, EPI, 2, 1>(p, (M + 31) / 32, N, st);
 }
