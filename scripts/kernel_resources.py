@@ -7,7 +7,8 @@ from pathlib import Path
 
 root = Path(__file__).resolve().parents[1]
 src = sys.argv[1]
-cmd = ["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC",
+cmd = ["/opt/rocm/bin/hipcc", "--offload-arch=gfx950", "-Xclang", "-target-feature",
+       "-Xclang", "-packed-fp32-ops", "-O3", "-std=c++17", "-fPIC",
        f"-I{root / 'include'}",
        f"-I{root / 'pagedattention-based-transformer-decoder-inference-framework_amd' / 'csrc'}",
        "-c", src, "-o", "/tmp/_kr.o", "-Rpass-analysis=kernel-resource-usage"]
