@@ -115,6 +115,87 @@ def moe(h, w, mlp):
     return out
 
 
+def rotate_pairs(x, positions, rot):
+    """x [T][heads][dim]: pairs (2i, 2i + 1) of the first dims dimensions turned."""
+    f, mul = rope_frequencies(rot)
+    a = positions[:, None].astype(np.float64) * f
+    c, s = (np.cos(a) * mul)[:, None, :], (np.sin(a) * mul)[:, None, :]
+    c, s = c.astype(x.dtype), s.astype(x.dtype)
+    n = rot["dims"]
+    u, v = x[..., 0:n:2], x[..., 1:n:2]
+    out = x.copy()
+    out[..., 0:n:2] = u * c - v * s
+    out[..., 1:n:2] = v * c + u * s
+    return out
+
+
+def latent_attention(h, w, mixer, positions, eps):
+    """Causal attention whose keys and values are products of one normed latent
+    per token; a rotated key part is shared by the heads."""
+    T = h.shape[0]
+    H, D, Dr, Dv, R = (mixer[k] for k in ("heads", "dim", "rot_dim", "vdim", "kv_rank"))
+    rot = dict(mixer["rot"], dims=Dr)
+    q = (h @ w["q"].T).reshape(T, H, D + Dr)
+    down = h @ w["dkv"].T
+    c = rms_norm(down[:, :R], w["dkv.norm"], eps)
+    k_rot = rotate_pairs(down[:, None, R:], positions, rot)[:, 0]
+    q_rot = rotate_pairs(q[..., D:], positions, rot)
+    k = (c @ w["uk"].T).reshape(T, H, D)
+    v = (c @ w["uv"].T).reshape(T, H, Dv)
+    out = np.empty((T, H, Dv), h.dtype)
+    for b in range(0, T, 256):
+        s = np.matmul(q[b:b + 256, :, :D].transpose(1, 0, 2), k.transpose(1, 2, 0))
+        s = (s + np.matmul(q_rot[b:b + 256].transpose(1, 0, 2), k_rot.T)) * mixer["scale"]
+        s = np.where(positions[None, None, :] <= positions[None, b:b + 256, None], s, -np.inf)
+        out[b:b + 256] = np.matmul(sink_softmax(s, w.get("sink")),
+                                   v.transpose(1, 0, 2)).transpose(1, 0, 2)
+    return out.reshape(T, H * Dv) @ w["o"].T
+
+
+def silu(x):
+    return x / (1 + np.exp(-x))
+
+
+def causal_conv(x, taps, bias):
+    """x [T][channels], taps [channels][n]: the last tap meets the current token,
+    zeros stand before the first."""
+    n = taps.shape[1]
+    padded = np.concatenate([np.zeros((n - 1, x.shape[1]), x.dtype), x])
+    return sum(padded[k:k + len(x)] * taps[:, k] for k in range(n)) + bias
+
+
+def selective_scan(x, dt, A, B, C, D):
+    """S <- exp(dt A) S + dt x B, y = S C + D x, token by token from S = 0.
+    x, dt [T][channels], A [channels][state], B, C [T][state], D [channels]."""
+    S = np.zeros(A.shape, x.dtype)
+    y = np.empty_like(x)
+    for t in range(len(x)):
+        S = np.exp(dt[t][:, None] * A) * S + (dt[t] * x[t])[:, None] * B[t]
+        y[t] = S @ C[t] + D * x[t]
+    return y
+
+
+def mamba1(h, w, mixer):
+    inner, rank, state = mixer["inner"], mixer["dt_rank"], mixer["state"]
+    xz = h @ w["in"].T
+    x, z = xz[:, :inner], xz[:, inner:]
+    x = silu(causal_conv(x, w["conv"], w["conv.b"]))
+    low = x @ w["x"].T
+    dt = np.logaddexp(0, low[:, :rank] @ w["dt"].T + w["dt.b"])
+    y = selective_scan(x, dt, -np.exp(w["A_log"]), low[:, rank:rank + state],
+                       low[:, rank + state:], w["D"])
+    return (y * silu(z)) @ w["o"].T
+
+
+def mix_streams(x, y, hc_mix, hc_out):
+    """x [streams][T][width] -> sum over s of mix[s, t] x_s + out[t] y."""
+    return np.tensordot(hc_mix.T, x, 1) + hc_out[:, None, None] * y
+
+
+def softcap(x, cap):
+    return cap * np.tanh(x / cap)
+
+
 def layer_runs(cfg):
     """[(layer, first layer of a repeated pass?)] in the order they run."""
     n = len(cfg["layers"])
@@ -158,3 +239,42 @@ def forward(cfg, weights, tokens, dtype=np.float64, taps=None):
         if taps is not None:
             taps.append(x)
     return rms_norm(x, get("final.norm"), eps) @ get("head").T
+
+
+def forward_streams(cfg, weights, tokens, dtype=np.float64, taps=None):
+    """Logits [T][vocab] of a model with several residual streams (Nubosun)."""
+    cache = {}
+
+    def get(name):
+        if name not in cache:
+            cache[name] = np.asarray(weights[name]).astype(dtype)
+        return cache[name]
+
+    def sub(prefix):
+        return {n[len(prefix):]: get(n) for n in weights if n.startswith(prefix)}
+
+    eps = cfg["norm"]["eps"]
+    positions = np.arange(len(tokens))
+    emb = get("embed")[np.asarray(tokens)] * dtype(cfg["embedding"]["scale"])
+    x = np.repeat(emb[None], cfg["streams"], 0)
+
+    def sublayer(x, p, q, f):
+        u = np.tensordot(get(f"{p}hc{q}.in"), x, 1)
+        y = f(rms_norm(u, get(f"{p}norm{q}"), eps)) * get(f"{p}ls{q}")
+        return mix_streams(x, y, get(f"{p}hc{q}.mix"), get(f"{p}hc{q}.out"))
+
+    for i, _ in layer_runs(cfg):
+        L, p = cfg["layers"][i], f"l{i}."
+        w = sub(p + "mix.")
+        if L["type"] == "mamba1":
+            x = sublayer(x, p, 1, lambda h: mamba1(h, w, L["mixer"]))
+        else:
+            x = sublayer(x, p, 1, lambda h: latent_attention(h, w, L["mixer"], positions, eps))
+        if L.get("mlp"):
+            m = sub(p + "mlp.")
+            x = sublayer(x, p, 2, lambda h: clamped_glu(h, m["gate"], m["up"], m["down"],
+                                                        L["mlp"]["limit"]))
+        if taps is not None:
+            taps.append(x.sum(0))
+    z = rms_norm(x.sum(0), get("final.norm"), eps) @ get("head").T
+    return softcap(z, cfg["logit_softcap"]) if cfg.get("logit_softcap") else z

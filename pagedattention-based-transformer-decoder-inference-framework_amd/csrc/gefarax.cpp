@@ -1,41 +1,13 @@
 // The Gefarax family: config.json -> LayerStackConfig.
-#include <cmath>
-
 #include "common.hpp"
-#include "layer_stack.hpp"
+#include "config_reader.hpp"
 
 namespace llm {
 namespace {
 
-constexpr float kGluAlpha = 1.702f;
-constexpr float kGluUpBias = 1.f;
-
-struct Reader {
-  std::string error;
-  double num(const Json& o, const char* key, const std::string& where) {
-    const Json& v = o[key];
-    if (v.kind != Json::Number && error.empty())
-      error = "config.json: " + where + "." + key + " is missing or not a number";
-    return v.num;
-  }
-  int size(const Json& o, const char* key, const std::string& where) {
-    const double d = num(o, key, where);
-    if (error.empty() && (d < 0 || d > 1e9 || d != std::floor(d)))
-      error = "config.json: " + where + "." + key + " is not a size";
-    return (int)d;
-  }
-};
-
-void read_expert(Reader& r, const Json& j, const std::string& where, ExpertSpec* e) {
-  e->ff = r.size(j, "ff", where);
-  e->glu.limit = (float)r.num(j, "limit", where);
-  e->glu.alpha = kGluAlpha;
-  e->glu.up_bias = kGluUpBias;
-}
-
 int make_gefarax(const Json& c, const std::string& dir, const ModelOptions& opt,
                  std::unique_ptr<StepModel>* out) {
-  Reader r;
+  ConfigReader r;
   LayerStackConfig cfg;
   cfg.vocab = r.size(c, "vocab", "config");
   cfg.width = r.size(c, "width", "config");
@@ -56,16 +28,7 @@ int make_gefarax(const Json& c, const std::string& dir, const ModelOptions& opt,
     if (m.has("rot")) {
       const Json& rot = m["rot"];
       s.attn.rope.dims = r.size(rot, "dims", at + ".mixer.rot");
-      s.attn.rope.base = r.num(rot, "base", at + ".mixer.rot");
-      if (rot.has("scaling")) {
-        const Json& sc = rot["scaling"];
-        const std::string w = at + ".mixer.rot.scaling";
-        s.attn.rope.yarn = true;
-        s.attn.rope.factor = r.num(sc, "factor", w);
-        s.attn.rope.original = r.num(sc, "original", w);
-        s.attn.rope.fast = r.num(sc, "fast", w);
-        s.attn.rope.slow = r.num(sc, "slow", w);
-      }
+      r.rope(rot, at + ".mixer.rot", &s.attn.rope);
     }
     if (l.has("mlp")) {
       const Json& f = l["mlp"];
@@ -76,19 +39,17 @@ int make_gefarax(const Json& c, const std::string& dir, const ModelOptions& opt,
       s.moe.experts = r.size(f["router"], "experts", w + ".router");
       s.moe.top = r.size(f["router"], "top", w + ".router");
       s.moe.scale = (float)r.num(f["router"], "scale", w + ".router");
-      read_expert(r, f["expert"], w + ".expert", &s.moe.expert);
+      r.glu(f["expert"], w + ".expert", &s.moe.expert);
       if (f.has("shared")) {
         s.moe.has_shared = true;
-        read_expert(r, f["shared"], w + ".shared", &s.moe.shared);
+        r.glu(f["shared"], w + ".shared", &s.moe.shared);
       }
     }
     cfg.layers.push_back(s);
   }
-  if (c.has("loop")) {
-    cfg.loop_start = r.size(c["loop"], "start", "loop");
-    cfg.loop_stop = r.size(c["loop"], "stop", "loop");
-    cfg.loop_times = r.size(c["loop"], "times", "loop");
-  }
+  r.loop(c, &cfg);
+  cfg.loop_adds_embedding = true;
+  cfg.post_norm = true;
   if (!r.error.empty()) return fail(LLM_ERR_INVALID, r.error);
   return make_layer_stack(cfg, dir, opt, out);
 }

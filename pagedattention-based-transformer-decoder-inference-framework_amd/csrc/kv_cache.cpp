@@ -60,7 +60,7 @@ int KvCache::init(int L_, int beams_, int H_, int D_, int TS_, int max_tiles_, l
   L = L_; beams = beams_; H = H_; D = D_; TS = TS_; max_tiles = max_tiles_; num_pages = pages;
   dtype = dtype_;
   es = dtype == LLM_F32 ? 4 : dtype == LLM_I8 ? 1 : 2;
-  Dv = Dv_ > 0 ? Dv_ : D;
+  Dv = Dv_ > 0 ? Dv_ : Dv_ < 0 ? 0 : D;
   page_elems = (size_t)TS * D;
   v_page_elems = (size_t)TS * Dv;
   // A wave loads K page p and V page p together.  With two separate pools at

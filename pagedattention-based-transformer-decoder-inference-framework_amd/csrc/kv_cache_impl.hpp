@@ -17,7 +17,7 @@ namespace llm {
 
 struct KvCache {
   int L = 0, beams = 0, H = 0, D = 0, TS = 0, max_tiles = 0;
-  int Dv = 0;  // value head size (D unless init was given another)
+  int Dv = 0;  // value head size (D unless init was given another; 0: no value pages)
   long long num_pages = 0;
   int dtype = LLM_F16;  // pool element type
   int es = 2;           // bytes per element
@@ -61,6 +61,7 @@ struct KvCache {
   bool lru_evict_one();  // false: nothing left to evict
 
   ~KvCache();
+  // Dv: 0 = as D, negative = keys only (latents that serve as keys and values)
   int init(int L, int beams, int H, int D, int TS, int max_tiles, long long pages,
            int dtype = LLM_F16, int Dv = 0);
   // zero the pools (layouts that pad their rows rely on zero padding)

@@ -2,33 +2,30 @@
 //
 // One step runs every entry of a mixed batch (prompt portions beside single
 // decoded tokens) as one list of token rows:
-//   angles | embed + norm -> per layer run { q|k|v product, rotation, append to
-//   the pages -> paged attention -> o product -> add + norm -> router product ->
-//   routing -> grouped gate/up product -> grouped down product -> add + norm }
-//   -> norm of the wanted rows -> head product.
+//   angles | embed + norm -> per layer run { mixer -> add + norm -> feed-forward
+//   -> add + norm } -> norm of the wanted rows -> head product
+// where a mixer is one of
+//   attention: q|k|v product, rotation, append to the pages -> paged attention ->
+//     o product
+//   latent attention (mix_latent.cpp), selective scan (mix_mamba.cpp)
+// and the feed-forward a gated pair of products, dense or of routed experts.
 // Everything a step depends on besides the weights is in one device block
 // (tokens, positions, slots, attention items, wanted rows) written by one copy,
 // so a decode step's launches are captured into a hipGraph per shape and
 // replayed.
 //
-// The cache: layers of one (kv_heads, dim, vdim) share a KvCache; each run of a
-// layer is a cache layer of its own, so a repeated layer keeps one cache per
-// pass.
-#include "layer_stack.hpp"
+// The cache: layers of one head geometry share a KvCache; each run of a layer is
+// a cache layer of its own (or has a StateCache of its own), so a repeated layer
+// keeps one cache or state per pass.
+#include "layer_stack_impl.hpp"
 
 #include <algorithm>
 #include <cmath>
 #include <cstring>
-#include <map>
 #include <mutex>
 
 #include "common.hpp"
-#include "dev_buf.hpp"
-#include "kv_cache_impl.hpp"
-#include "moe.hpp"
-#include "paged_gqa.hpp"
-#include "rms_norm.hpp"
-#include "safetensors.hpp"
+#include "paged_latent.hpp"
 
 namespace llm {
 
@@ -71,19 +68,41 @@ int check_config(const LayerStackConfig& c, const ModelOptions& o) {
   LLM_REQUIRE(c.loop_times >= 1 && c.loop_start >= 0 && c.loop_start <= c.loop_stop &&
                   c.loop_stop <= (int)c.layers.size(),
               "config: bad loop");
+  LLM_REQUIRE(c.streams >= 0 && c.streams <= kMaxStreams, "config: streams must be at most " +
+                                                              std::to_string(kMaxStreams));
+  const auto rope_ok = [](const RopeSpec& r) {
+    return r.dims >= 0 && r.dims % 2 == 0 && (r.dims == 0 || r.base > 1.0);
+  };
   for (size_t i = 0; i < c.layers.size(); ++i) {
-    const AttentionSpec& a = c.layers[i].attn;
+    const LayerSpec& l = c.layers[i];
     const std::string at = "config: layer " + std::to_string(i) + ": ";
-    LLM_REQUIRE(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0,
-                at + "heads must be a multiple of kv_heads");
-    LLM_REQUIRE(a.dim > 0 && a.vdim > 0 && a.dim <= kGqaMaxDim && a.vdim <= kGqaMaxDim &&
-                    a.dim % 2 == 0,
-                at + "head sizes must be in [1, 256] and dim even");
-    LLM_REQUIRE(a.rope.dims >= 0 && a.rope.dims <= a.dim && a.rope.dims % 2 == 0 &&
-                    (a.rope.dims == 0 || a.rope.base > 1.0),
-                at + "rot.dims must be even and at most dim, rot.base > 1");
-    if (!c.layers[i].has_mlp) continue;
-    const MoeSpec& m = c.layers[i].moe;
+    if (l.mixer == Mixer::kAttention) {
+      const AttentionSpec& a = l.attn;
+      LLM_REQUIRE(a.heads > 0 && a.kv_heads > 0 && a.heads % a.kv_heads == 0,
+                  at + "heads must be a multiple of kv_heads");
+      LLM_REQUIRE(a.dim > 0 && a.vdim > 0 && a.dim <= kGqaMaxDim && a.vdim <= kGqaMaxDim &&
+                      a.dim % 2 == 0,
+                  at + "head sizes must be in [1, 256] and dim even");
+      LLM_REQUIRE(rope_ok(a.rope) && a.rope.dims <= a.dim,
+                  at + "rot.dims must be even and at most dim, rot.base > 1");
+    } else if (l.mixer == Mixer::kLatent) {
+      const LatentSpec& a = l.latent;
+      LLM_REQUIRE(a.heads > 0 && a.dim > 0 && a.vdim > 0 && a.rank > 0,
+                  at + "heads, dim, vdim and kv_rank must be positive");
+      LLM_REQUIRE(rope_ok(a.rope), at + "rot_dim must be even, rot.base > 1");
+      LLM_REQUIRE(a.rank <= kLatentMaxRank && latent_row(a.rank, a.rot_dim) <= kLatentMaxRow,
+                  at + "kv_rank is at most 512, with rot_dim at most 576");
+    } else {
+      const MambaSpec& m = l.mamba;
+      LLM_REQUIRE(m.inner > 0 && m.dt_rank > 0 && m.taps > 0 && m.state > 0 && m.state <= kMaxScanState,
+                  at + "inner, dt_rank and conv must be positive, state in [1, 256]");
+    }
+    if (!l.has_mlp) continue;
+    if (l.dense) {
+      LLM_REQUIRE(l.ffn.ff >= 1, at + "mlp.ff must be positive");
+      continue;
+    }
+    const MoeSpec& m = l.moe;
     LLM_REQUIRE(m.experts >= 1 && m.experts <= kMaxExperts && m.top >= 1 && m.top <= m.experts &&
                     m.expert.ff >= 1 && (!m.has_shared || m.shared.ff >= 1),
                 at + "bad expert sizes");
@@ -91,139 +110,7 @@ int check_config(const LayerStackConfig& c, const ModelOptions& o) {
   return LLM_OK;
 }
 
-inline int up(int v, int m) { return (v + m - 1) / m * m; }
-
-class LayerStack final : public StepModel {
- public:
-  ~LayerStack() override {
-    if (meta_done_) (void)hipEventSynchronize(meta_done_);
-    clear_graphs();
-    if (h_meta_) (void)hipHostFree(h_meta_);
-    if (meta_done_) (void)hipEventDestroy(meta_done_);
-    if (cap_stream_) (void)hipStreamDestroy(cap_stream_);
-  }
-  int init(const LayerStackConfig& cfg, const std::string& dir, const ModelOptions& opt);
-
-  int vocab() const override { return cfg_.vocab; }
-  int max_seq_len() const override { return max_len_; }
-  int max_step_tokens() const override { return cap_; }
-  int page_tokens() const override { return kPageTokens; }
-  long long pool_tokens() const override { return pool_pages_ * kPageTokens; }
-  long long free_tokens() const override {
-    long long n = pool_pages_;
-    for (const auto& g : geos_) n = std::min(n, g->kv.free_count() / ((long long)g->layers * g->G));
-    return n * kPageTokens;
-  }
-  int forward(const std::vector<StepSeq>& batch, float* logits, hipStream_t st) override;
-  int release(int slot) override;
-  int layer_runs() const override { return (int)runs_.size(); }
-  int width() const override { return cfg_.width; }
-  int set_tap(float* host) override {
-    tap_ = host;
-    return LLM_OK;
-  }
-
- private:
-  struct Geometry {  // cache of the layers of one head geometry
-    int G = 0, D = 0, Dv = 0, Dp = 0, Dvp = 0, layers = 0;
-    KvCache kv;
-  };
-  struct Run {
-    int layer = 0, geo = 0, cache_layer = 0;
-    bool add_embed = false;
-  };
-  struct Layer {
-    LayerSpec s;
-    int geo = 0, rope = -1, plan = 0;
-    DevBuf<float> norm1, norm1b, norm2, norm2b, sink, correction;
-    DevBuf<uint8_t> qkv, o, router, experts_in, experts_out, shared_in, shared_out;
-    DevBuf<MmGroup> groups;
-    int n_qkv = 0;
-  };
-  struct Rope {
-    RopeSpec spec;
-    float mul = 1.f;
-    DevBuf<float> freq;
-    DevBuf<float2> turn;
-  };
-  // one attention launch of the step: its items and merges in the meta block
-  struct Launch {
-    int tile_rows = 16, n_items = 0, n_merges = 0, parts = 0;
-    size_t items_at = 0, merges_at = 0;
-  };
-  struct Plan {  // layers that cut their rows alike
-    int R = 1, G = 1, big_rows = 16, max_pd = 16;
-    Launch small, big;
-  };
-
-  int load(const std::string& dir);
-  int pack_rows(const SafeTensors& f, const std::vector<std::pair<std::string, int>>& parts, int K,
-                const std::vector<int32_t>* map, uint8_t* dst);
-  int ensure_rows(int M);
-  int build_meta(const std::vector<StepSeq>& batch, int M, int n_want, hipStream_t st);
-  void cut(const std::vector<StepSeq>& batch, Plan& p, bool big, std::vector<GqaItem>& items,
-           std::vector<GqaMerge>& merges, Launch& l);
-  int enqueue(int M, int n_want, float* logits, hipStream_t st);
-  int attention(const Layer& l, const Run& r, int M, hipStream_t st);
-  int mlp(const Layer& l, int M, hipStream_t st);
-  void clear_graphs() {
-    for (auto& g : graphs_)
-      if (g.second) (void)hipGraphExecDestroy(g.second);
-    graphs_.clear();
-  }
-
-  LayerStackConfig cfg_;
-  ModelOptions opt_;
-  int dt_ = LLM_BF16, es_ = 2, ldx_ = 0, cap_ = 0, max_len_ = 0, w_nt_ = 0;
-  long long pool_pages_ = 0;
-  std::vector<std::unique_ptr<Geometry>> geos_;
-  std::vector<std::unique_ptr<Layer>> layers_;
-  std::vector<std::unique_ptr<Rope>> ropes_;
-  std::vector<Run> runs_;
-  std::vector<Plan> plans_;
-  DevBuf<uint16_t> emb_;
-  DevBuf<float> final_norm_;
-  DevBuf<uint8_t> head_;
-  DevBuf<uint8_t> staging_;
-  DevBuf<int32_t> map_;
-  size_t weight_bytes_ = 0;
-
-  // step buffers, sized for rows_ tokens
-  int rows_ = 0;
-  int ld_q_ = 0, ld_att_ = 0, ld_act_ = 0, ld_shared_ = 0, max_top_ = 0, max_e_ = 0;
-  DevBuf<float> x_, y_, z_, weight_, part_o_, part_ml_;
-  DevBuf<uint8_t> h_, q_, att_, act_, act_shared_;
-  DevBuf<int32_t> choice_, perm_, n_tiles_;
-  DevBuf<MmTile> tiles_;
-  // the step's meta block
-  DevBuf<uint8_t> meta_;
-  uint8_t* h_meta_ = nullptr;
-  size_t meta_cap_ = 0;
-  hipEvent_t meta_done_ = nullptr;
-  size_t at_tok_ = 0, at_pos_ = 0, at_slot_ = 0, at_want_ = 0;
-  float* tap_ = nullptr;
-
-  bool use_graph_ = true;
-  hipStream_t cap_stream_ = nullptr;
-  std::map<std::vector<long long>, hipGraphExec_t> graphs_;  // NULL: seen once, not captured
-
-  template <typename T>
-  const T* meta(size_t at) const { return reinterpret_cast<const T*>(meta_.p + at); }
-};
-
-template <typename T>
-int alloc_zero(DevBuf<T>& b, size_t n) {
-  RET_IF(b.alloc(n));
-  if (n) LLM_HIP_RET(hipMemset(b.p, 0, n * sizeof(T)));
-  return LLM_OK;
-}
-
-template <typename T>
-int upload_vec(DevBuf<T>& b, const std::vector<T>& v) {
-  RET_IF(b.alloc(v.size()));
-  if (!v.empty()) LLM_HIP_RET(hipMemcpy(b.p, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice));
-  return LLM_OK;
-}
+}  // namespace
 
 int LayerStack::init(const LayerStackConfig& cfg, const std::string& dir, const ModelOptions& opt) {
   RET_IF(check_config(cfg, opt));
@@ -243,46 +130,27 @@ int LayerStack::init(const LayerStackConfig& cfg, const std::string& dir, const 
   for (const LayerSpec& s : cfg.layers) {
     auto l = std::make_unique<Layer>();
     l->s = s;
-    const AttentionSpec& a = s.attn;
-    int g = 0;
-    for (; g < (int)geos_.size(); ++g)
-      if (geos_[g]->G == a.kv_heads && geos_[g]->D == a.dim && geos_[g]->Dv == a.vdim) break;
-    if (g == (int)geos_.size()) {
-      auto n = std::make_unique<Geometry>();
-      n->G = a.kv_heads;
-      n->D = a.dim;
-      n->Dv = a.vdim;
-      n->Dp = up(a.dim, 8);
-      n->Dvp = up(a.vdim, 8);
-      geos_.push_back(std::move(n));
+    if (s.mixer == Mixer::kLatent) {
+      RET_IF(init_latent(*l));
+    } else if (s.mixer == Mixer::kMamba) {
+      RET_IF(init_mamba(*l));
+    } else {
+      const AttentionSpec& a = s.attn;
+      l->geo = find_geometry(false, a.kv_heads, a.dim, a.vdim);
+      const Geometry& geo = *geos_[l->geo];
+      RET_IF(find_rope(a.rope, &l->rope));
+      auto p = std::make_unique<Plan>();
+      p->R = a.heads / a.kv_heads;
+      p->G = a.kv_heads;
+      p->big_tile = gqa_tile_rows(dt_, geo.Dp, geo.Dvp, 1 << 20);
+      p->max_pd = gqa_part_dim(a.vdim);
+      l->plan = add_plan(std::move(p));
+      ld_q_ = std::max(ld_q_, a.heads * geo.Dp);
+      ld_att_ = std::max(ld_att_, mm_pad(a.heads * a.vdim));
     }
-    l->geo = g;
-    const Geometry& geo = *geos_[g];
-    if (a.rope.dims > 0) {
-      int r = 0;
-      for (; r < (int)ropes_.size(); ++r)
-        if (ropes_[r]->spec == a.rope) break;
-      if (r == (int)ropes_.size()) {
-        auto n = std::make_unique<Rope>();
-        n->spec = a.rope;
-        RET_IF(upload_vec(n->freq, rope_frequencies(a.rope, &n->mul)));
-        ropes_.push_back(std::move(n));
-      }
-      l->rope = r;
-    }
-    Plan p;
-    p.R = a.heads / a.kv_heads;
-    p.G = a.kv_heads;
-    p.big_rows = gqa_tile_rows(dt_, geo.Dp, geo.Dvp, 1 << 20);
-    int k = 0;
-    for (; k < (int)plans_.size(); ++k)
-      if (plans_[k].R == p.R && plans_[k].G == p.G && plans_[k].big_rows == p.big_rows) break;
-    if (k == (int)plans_.size()) plans_.push_back(p);
-    plans_[k].max_pd = std::max(plans_[k].max_pd, gqa_part_dim(a.vdim));
-    l->plan = k;
-    ld_q_ = std::max(ld_q_, a.heads * geo.Dp);
-    ld_att_ = std::max(ld_att_, mm_pad(a.heads * a.vdim));
-    if (s.has_mlp) {
+    if (s.has_mlp && s.dense) {
+      ld_act_ = std::max(ld_act_, mm_pad(s.ffn.ff));
+    } else if (s.has_mlp) {
       max_top_ = std::max(max_top_, s.moe.top);
       max_e_ = std::max(max_e_, s.moe.experts);
       ld_act_ = std::max(ld_act_, mm_pad(s.moe.expert.ff));
@@ -290,23 +158,15 @@ int LayerStack::init(const LayerStackConfig& cfg, const std::string& dir, const 
     }
     layers_.push_back(std::move(l));
   }
-  const auto add_run = [&](int i, bool again) {
-    Run r;
-    r.layer = i;
-    r.geo = layers_[i]->geo;
-    r.cache_layer = geos_[r.geo]->layers++;
-    r.add_embed = again;
-    runs_.push_back(r);
-  };
-  for (int i = 0; i < cfg.loop_start; ++i) add_run(i, false);
+  for (int i = 0; i < cfg.loop_start; ++i) RET_IF(add_run(i, false));
   for (int p = 0; p < cfg.loop_times; ++p)
-    for (int i = cfg.loop_start; i < cfg.loop_stop; ++i) add_run(i, p > 0 && i == cfg.loop_start);
-  for (int i = cfg.loop_stop; i < (int)layers_.size(); ++i) add_run(i, false);
+    for (int i = cfg.loop_start; i < cfg.loop_stop; ++i) RET_IF(add_run(i, p > 0 && i == cfg.loop_start));
+  for (int i = cfg.loop_stop; i < (int)layers_.size(); ++i) RET_IF(add_run(i, false));
 
   for (auto& g : geos_) {
     if (g->layers == 0) continue;
     RET_IF(g->kv.init(g->layers, opt.max_seqs, g->G, g->Dp, kPageTokens, max_len_ / kPageTokens,
-                      pool_pages_ * g->layers * g->G, dt_, g->Dvp));
+                      pool_pages_ * g->layers * g->G, dt_, g->latent ? -1 : g->Dvp));
     RET_IF(g->kv.zero_pools(nullptr));
   }
   LLM_HIP_RET(hipEventCreateWithFlags(&meta_done_, hipEventDisableTiming));
@@ -316,12 +176,68 @@ int LayerStack::init(const LayerStackConfig& cfg, const std::string& dir, const 
   return LLM_OK;
 }
 
+int LayerStack::find_rope(const RopeSpec& spec, int* index) {
+  *index = -1;
+  if (spec.dims == 0) return LLM_OK;
+  int r = 0;
+  for (; r < (int)ropes_.size(); ++r)
+    if (ropes_[r]->spec == spec) break;
+  if (r == (int)ropes_.size()) {
+    auto n = std::make_unique<Rope>();
+    n->spec = spec;
+    RET_IF(upload_vec(n->freq, rope_frequencies(spec, &n->mul)));
+    ropes_.push_back(std::move(n));
+  }
+  *index = r;
+  return LLM_OK;
+}
+
+int LayerStack::find_geometry(bool latent, int G, int D, int Dv) {
+  for (size_t g = 0; g < geos_.size(); ++g)
+    if (geos_[g]->latent == latent && geos_[g]->G == G && geos_[g]->D == D && geos_[g]->Dv == Dv)
+      return (int)g;
+  auto n = std::make_unique<Geometry>();
+  n->latent = latent;
+  n->G = G;
+  n->D = D;
+  n->Dv = Dv;
+  n->Dp = latent ? latent_row(D, Dv) : up(D, 8);
+  n->Dvp = latent ? 0 : up(Dv, 8);
+  geos_.push_back(std::move(n));
+  return (int)geos_.size() - 1;
+}
+
+int LayerStack::add_plan(std::unique_ptr<Plan> p) {
+  size_t k = 0;
+  for (; k < plans_.size(); ++k)
+    if (plans_[k]->same(*p)) break;
+  const int pd = p->max_pd;
+  if (k == plans_.size()) plans_.push_back(std::move(p));
+  plans_[k]->max_pd = std::max(plans_[k]->max_pd, pd);
+  return (int)k;
+}
+
+int LayerStack::add_run(int layer, bool again) {
+  const Layer& l = *layers_[layer];
+  Run r;
+  r.layer = layer;
+  r.again = again;
+  if (l.geo >= 0) r.cache_layer = geos_[l.geo]->layers++;
+  if (l.s.mixer == Mixer::kMamba) {
+    const MambaSpec& m = l.s.mamba;
+    r.state = std::make_unique<StateCache>();
+    RET_IF(r.state->init(opt_.max_seqs, m.state, mm_pad(m.inner), m.taps, es_));
+  }
+  runs_.push_back(std::move(r));
+  return LLM_OK;
+}
+
 // ---------------------------------------------------------------------------
 // weights
 // ---------------------------------------------------------------------------
 
 // Pack the rows of one or more [rows][K] tensors, stacked and then reordered by
-// `map` (packed column n takes stacked row map[n]).
+// `map` (packed column n takes stacked row map[n], zeros where it is -1).
 int LayerStack::pack_rows(const SafeTensors& f,
                           const std::vector<std::pair<std::string, int>>& parts, int K,
                           const std::vector<int32_t>* map, uint8_t* dst) {
@@ -338,7 +254,10 @@ int LayerStack::pack_rows(const SafeTensors& f,
     LLM_HIP_RET(hipMemcpy(staging_.p + at, t.data, t.bytes, hipMemcpyHostToDevice));
     at += t.bytes;
   }
-  if (map) RET_IF(upload_vec(map_, *map));
+  if (map) {
+    N = (int)map->size();
+    RET_IF(upload_vec(map_, *map));
+  }
   LLM_HIP_RET(mm_pack(dt_, reinterpret_cast<const uint16_t*>(staging_.p), map ? map_.p : nullptr, N,
                       K, dst, nullptr));
   LLM_HIP_RET(hipStreamSynchronize(nullptr));  // staging and map are used again
@@ -346,23 +265,57 @@ int LayerStack::pack_rows(const SafeTensors& f,
   return LLM_OK;
 }
 
+int LayerStack::pack_host(const std::vector<uint16_t>& rows, int K, const std::vector<int32_t>* map,
+                          uint8_t* dst) {
+  const size_t need = rows.size() * 2;
+  if (staging_.n < need) RET_IF(staging_.alloc(need));
+  LLM_HIP_RET(hipMemcpy(staging_.p, rows.data(), need, hipMemcpyHostToDevice));
+  const int N = map ? (int)map->size() : (int)(rows.size() / K);
+  if (map) RET_IF(upload_vec(map_, *map));
+  LLM_HIP_RET(mm_pack(dt_, reinterpret_cast<const uint16_t*>(staging_.p), map ? map_.p : nullptr, N,
+                      K, dst, nullptr));
+  LLM_HIP_RET(hipStreamSynchronize(nullptr));
+  weight_bytes_ += mm_packed_bytes(dt_, N, K);
+  return LLM_OK;
+}
+
+int LayerStack::load_packed(const SafeTensors& f,
+                            const std::vector<std::pair<std::string, int>>& parts, int K,
+                            const std::vector<int32_t>* map, DevBuf<uint8_t>& b) {
+  int N = 0;
+  for (const auto& p : parts) N += p.second;
+  RET_IF(b.alloc(mm_packed_bytes(dt_, map ? (int)map->size() : N, K)));
+  return pack_rows(f, parts, K, map, b.p);
+}
+
+int LayerStack::load_vector(const SafeTensors& f, const std::string& name, int n, int padded,
+                            DevBuf<float>& b) {
+  std::vector<float> v;
+  RET_IF(f.get_f32(name, {n}, &v));
+  v.resize(padded, 0.f);
+  return upload_vec(b, v);
+}
+
+int LayerStack::load_hyper(const SafeTensors& f, const std::string& name, Hyper& h) {
+  const int S = cfg_.streams;
+  std::vector<float> v;
+  RET_IF(load_vector(f, name + ".in", S, S, h.in));
+  RET_IF(load_vector(f, name + ".out", S, S, h.out));
+  RET_IF(f.get_f32(name + ".mix", {S, S}, &v));
+  return upload_vec(h.mix, v);
+}
+
+// column 2i: gate i, 2i + 1: up i
+static std::vector<int32_t> gate_up_rows(int ff) {
+  std::vector<int32_t> v((size_t)2 * ff);
+  for (int n = 0; n < 2 * ff; ++n) v[n] = (n & 1) * ff + n / 2;
+  return v;
+}
+
 int LayerStack::load(const std::string& dir) {
   SafeTensors f;
   RET_IF(f.open(dir + "/model.safetensors"));
   const int W = cfg_.width;
-  const auto padded = [&](DevBuf<float>& b, const std::string& name) {
-    std::vector<float> v;
-    RET_IF(f.get_f32(name, {W}, &v));
-    v.resize(ldx_, 0.f);
-    return upload_vec(b, v);
-  };
-  const auto packed = [&](DevBuf<uint8_t>& b, const std::vector<std::pair<std::string, int>>& parts,
-                          int K, const std::vector<int32_t>* map) {
-    int N = 0;
-    for (const auto& p : parts) N += p.second;
-    RET_IF(b.alloc(mm_packed_bytes(dt_, N, K)));
-    return pack_rows(f, parts, K, map, b.p);
-  };
   {
     std::vector<uint16_t> e;
     RET_IF(f.get_bf16("embed", {cfg_.vocab, W}, &e));
@@ -374,76 +327,90 @@ int LayerStack::load(const std::string& dir) {
   for (size_t i = 0; i < layers_.size(); ++i) {
     Layer& l = *layers_[i];
     const std::string at = "l" + std::to_string(i) + ".", mix = at + "mix.", ml = at + "mlp.";
-    const AttentionSpec& a = l.s.attn;
-    RET_IF(padded(l.norm1, at + "norm1"));
-    RET_IF(padded(l.norm1b, at + "norm1b"));
-    // q | k | v with rotation partners side by side
-    const int nq = a.heads * a.dim, nk = a.kv_heads * a.dim, nv = a.kv_heads * a.vdim;
-    l.n_qkv = nq + nk + nv;
-    std::vector<int32_t> map((size_t)l.n_qkv);
-    const int half = a.rope.dims / 2;
-    for (int n = 0; n < l.n_qkv; ++n) {
-      const int d = n % a.dim;
-      map[n] = n < nq + nk && d < a.rope.dims ? n - d + d / 2 + (d & 1) * half : n;
-    }
-    RET_IF(packed(l.qkv, {{mix + "q", nq}, {mix + "k", nk}, {mix + "v", nv}}, W, &map));
-    RET_IF(packed(l.o, {{mix + "o", W}}, a.heads * a.vdim, nullptr));
-    if (a.sink) {
-      std::vector<float> s;
-      RET_IF(f.get_f32(mix + "sink", {a.heads}, &s));
-      RET_IF(upload_vec(l.sink, s));
+    RET_IF(load_vector(f, at + "norm1", W, ldx_, l.norm1));
+    if (cfg_.post_norm) RET_IF(load_vector(f, at + "norm1b", W, ldx_, l.norm1b));
+    if (cfg_.layer_scale) RET_IF(load_vector(f, at + "ls1", W, ldx_, l.ls1));
+    if (cfg_.streams > 0) RET_IF(load_hyper(f, at + "hc1", l.hc1));
+    switch (l.s.mixer) {
+      case Mixer::kAttention: RET_IF(load_attention(f, mix, l)); break;
+      case Mixer::kLatent: RET_IF(load_latent(f, mix, l)); break;
+      case Mixer::kMamba: RET_IF(load_mamba(f, mix, l)); break;
     }
     if (!l.s.has_mlp) continue;
-    RET_IF(padded(l.norm2, at + "norm2"));
-    RET_IF(padded(l.norm2b, at + "norm2b"));
-    const MoeSpec& m = l.s.moe;
-    RET_IF(packed(l.router, {{ml + "router", m.experts}}, W, nullptr));
-    std::vector<float> c;
-    RET_IF(f.get_f32(ml + "correction", {m.experts}, &c));
-    RET_IF(upload_vec(l.correction, c));
-    const auto interleaved = [](int ff) {  // column 2i: gate i, 2i + 1: up i
-      std::vector<int32_t> v((size_t)2 * ff);
-      for (int n = 0; n < 2 * ff; ++n) v[n] = (n & 1) * ff + n / 2;
-      return v;
-    };
-    const auto describe = [&](const ExpertSpec& e, const uint8_t* in, const uint8_t* out) {
-      MmGroup g;
-      g.w_in = in;
-      g.w_out = out;
-      g.n_in = 2 * e.ff;
-      g.ks_in = (W + mm_kstep(dt_) - 1) / mm_kstep(dt_);
-      g.n_out = W;
-      g.ks_out = (e.ff + mm_kstep(dt_) - 1) / mm_kstep(dt_);
-      g.glu = e.glu;
-      return g;
-    };
-    std::vector<MmGroup> groups;
-    const int ff = m.expert.ff;
-    const size_t b_in = mm_packed_bytes(dt_, 2 * ff, W), b_out = mm_packed_bytes(dt_, W, ff);
-    RET_IF(l.experts_in.alloc(b_in * m.experts));
-    RET_IF(l.experts_out.alloc(b_out * m.experts));
-    const std::vector<int32_t> pairs = interleaved(ff);
-    for (int e = 0; e < m.experts; ++e) {
-      const std::string ex = ml + "e" + std::to_string(e) + ".";
-      uint8_t *in = l.experts_in.p + b_in * e, *out = l.experts_out.p + b_out * e;
-      RET_IF(pack_rows(f, {{ex + "gate", ff}, {ex + "up", ff}}, W, &pairs, in));
-      RET_IF(pack_rows(f, {{ex + "down", W}}, ff, nullptr, out));
-      groups.push_back(describe(m.expert, in, out));
+    RET_IF(load_vector(f, at + "norm2", W, ldx_, l.norm2));
+    if (cfg_.post_norm) RET_IF(load_vector(f, at + "norm2b", W, ldx_, l.norm2b));
+    if (cfg_.layer_scale) RET_IF(load_vector(f, at + "ls2", W, ldx_, l.ls2));
+    if (cfg_.streams > 0) RET_IF(load_hyper(f, at + "hc2", l.hc2));
+    if (l.s.dense) {
+      const int ff = l.s.ffn.ff;
+      const std::vector<int32_t> pairs = gate_up_rows(ff);
+      RET_IF(load_packed(f, {{ml + "gate", ff}, {ml + "up", ff}}, W, &pairs, l.ffn_in));
+      RET_IF(load_packed(f, {{ml + "down", W}}, ff, nullptr, l.ffn_out));
+    } else {
+      RET_IF(load_moe(f, ml, l));
     }
-    if (m.has_shared) {
-      const int sf = m.shared.ff;
-      const std::vector<int32_t> sp = interleaved(sf);
-      RET_IF(packed(l.shared_in, {{ml + "shared.gate", sf}, {ml + "shared.up", sf}}, W, &sp));
-      RET_IF(packed(l.shared_out, {{ml + "shared.down", W}}, sf, nullptr));
-      groups.push_back(describe(m.shared, l.shared_in.p, l.shared_out.p));
-    }
-    RET_IF(upload_vec(l.groups, groups));
   }
-  RET_IF(padded(final_norm_, "final.norm"));
-  RET_IF(packed(head_, {{"head", cfg_.vocab}}, W, nullptr));
+  RET_IF(load_vector(f, "final.norm", W, ldx_, final_norm_));
+  RET_IF(load_packed(f, {{"head", cfg_.vocab}}, W, nullptr, head_));
   RET_IF(staging_.alloc(0));
   RET_IF(map_.alloc(0));
   return LLM_OK;
+}
+
+int LayerStack::load_attention(const SafeTensors& f, const std::string& mix, Layer& l) {
+  const AttentionSpec& a = l.s.attn;
+  // q | k | v with rotation partners side by side
+  const int nq = a.heads * a.dim, nk = a.kv_heads * a.dim, nv = a.kv_heads * a.vdim;
+  l.n_qkv = nq + nk + nv;
+  std::vector<int32_t> map((size_t)l.n_qkv);
+  const int half = a.rope.dims / 2;
+  for (int n = 0; n < l.n_qkv; ++n) {
+    const int d = n % a.dim;
+    map[n] = n < nq + nk && d < a.rope.dims ? n - d + d / 2 + (d & 1) * half : n;
+  }
+  RET_IF(load_packed(f, {{mix + "q", nq}, {mix + "k", nk}, {mix + "v", nv}}, cfg_.width, &map, l.qkv));
+  RET_IF(load_packed(f, {{mix + "o", cfg_.width}}, a.heads * a.vdim, nullptr, l.o));
+  if (a.sink) RET_IF(load_vector(f, mix + "sink", a.heads, a.heads, l.sink));
+  return LLM_OK;
+}
+
+int LayerStack::load_moe(const SafeTensors& f, const std::string& ml, Layer& l) {
+  const MoeSpec& m = l.s.moe;
+  const int W = cfg_.width;
+  RET_IF(load_packed(f, {{ml + "router", m.experts}}, W, nullptr, l.router));
+  RET_IF(load_vector(f, ml + "correction", m.experts, m.experts, l.correction));
+  const auto describe = [&](const ExpertSpec& e, const uint8_t* in, const uint8_t* out) {
+    MmGroup g;
+    g.w_in = in;
+    g.w_out = out;
+    g.n_in = 2 * e.ff;
+    g.ks_in = (W + mm_kstep(dt_) - 1) / mm_kstep(dt_);
+    g.n_out = W;
+    g.ks_out = (e.ff + mm_kstep(dt_) - 1) / mm_kstep(dt_);
+    g.glu = e.glu;
+    return g;
+  };
+  std::vector<MmGroup> groups;
+  const int ff = m.expert.ff;
+  const size_t b_in = mm_packed_bytes(dt_, 2 * ff, W), b_out = mm_packed_bytes(dt_, W, ff);
+  RET_IF(l.experts_in.alloc(b_in * m.experts));
+  RET_IF(l.experts_out.alloc(b_out * m.experts));
+  const std::vector<int32_t> pairs = gate_up_rows(ff);
+  for (int e = 0; e < m.experts; ++e) {
+    const std::string ex = ml + "e" + std::to_string(e) + ".";
+    uint8_t *in = l.experts_in.p + b_in * e, *out = l.experts_out.p + b_out * e;
+    RET_IF(pack_rows(f, {{ex + "gate", ff}, {ex + "up", ff}}, W, &pairs, in));
+    RET_IF(pack_rows(f, {{ex + "down", W}}, ff, nullptr, out));
+    groups.push_back(describe(m.expert, in, out));
+  }
+  if (m.has_shared) {
+    const int sf = m.shared.ff;
+    const std::vector<int32_t> sp = gate_up_rows(sf);
+    RET_IF(load_packed(f, {{ml + "shared.gate", sf}, {ml + "shared.up", sf}}, W, &sp, l.shared_in));
+    RET_IF(load_packed(f, {{ml + "shared.down", W}}, sf, nullptr, l.shared_out));
+    groups.push_back(describe(m.shared, l.shared_in.p, l.shared_out.p));
+  }
+  return upload_vec(l.groups, groups);
 }
 
 // ---------------------------------------------------------------------------
@@ -457,14 +424,25 @@ int LayerStack::ensure_rows(int M) {
   LLM_HIP_RET(hipDeviceSynchronize());
   clear_graphs();
   rows_ = 0;
-  RET_IF(alloc_zero(x_, (size_t)n * ldx_));
+  RET_IF(alloc_zero(x_, (size_t)n * std::max(cfg_.streams, 1) * ldx_));
   RET_IF(alloc_zero(h_, (size_t)n * ldx_ * es_));
-  RET_IF(alloc_zero(q_, (size_t)n * ld_q_ * es_));
+  // (a product may read whole k-steps past the last row's end)
+  const size_t slack = (size_t)64 * es_;
+  RET_IF(alloc_zero(q_, (size_t)n * ld_q_ * es_ + slack));
   RET_IF(alloc_zero(att_, (size_t)n * ld_att_ * es_));
   RET_IF(alloc_zero(y_, (size_t)n * (max_top_ + 1) * ldx_));
+  RET_IF(alloc_zero(act_, (size_t)n * std::max(max_top_, 1) * ld_act_ * es_));
+  RET_IF(alloc_zero(q_lat_, (size_t)n * ld_qlat_ * es_ + slack));
+  RET_IF(alloc_zero(o_lat_, (size_t)n * ld_olat_ * es_ + slack));
+  RET_IF(alloc_zero(down_, (size_t)n * ld_down_));
+  RET_IF(alloc_zero(xz_, (size_t)n * ld_xz_ * es_));
+  RET_IF(alloc_zero(xc_, (size_t)n * ld_inner_ * es_));
+  RET_IF(alloc_zero(gated_, (size_t)n * ld_inner_ * es_));
+  RET_IF(alloc_zero(dtv_, (size_t)n * ld_inner_));
+  RET_IF(alloc_zero(low_, (size_t)n * ld_low_ * es_));
+  RET_IF(alloc_zero(bc_, (size_t)n * ld_bc_));
   if (max_top_ > 0) {
     RET_IF(alloc_zero(z_, (size_t)n * max_e_));
-    RET_IF(alloc_zero(act_, (size_t)n * max_top_ * ld_act_ * es_));
     RET_IF(alloc_zero(act_shared_, (size_t)n * ld_shared_ * es_));
     RET_IF(alloc_zero(weight_, (size_t)n * max_top_));
     RET_IF(alloc_zero(choice_, (size_t)n * max_top_));
@@ -478,18 +456,21 @@ int LayerStack::ensure_rows(int M) {
   return LLM_OK;
 }
 
-// The row tiles of one attention launch: sequences that bring few rows per
-// key/value head (big false) or many, split over their pages until the launch
+// The row tiles of one attention launch: the plan's sequences that bring few rows
+// per key/value head (big false) or many, split over their pages until the launch
 // holds about kTargetGroups workgroups; long tiles first.
 void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
                      std::vector<GqaItem>& items, std::vector<GqaMerge>& merges, Launch& l) {
   l = Launch();
-  l.tile_rows = big ? p.big_rows : 16;
+  l.tile_rows = big ? p.big_tile : p.small_tile;
+  const auto mine = [&](const StepSeq& s) {
+    return s.n >= p.min_n && s.n <= p.max_n && ((s.n * p.R > p.small_max) == big);
+  };
   long long tiles = 0;
-  int max_pages = 1, tok0 = 0;
+  int max_pages = 1, tok0 = 0, entry = 0;
   for (const StepSeq& s : batch) {
+    if (!mine(s)) continue;
     const int rows = s.n * p.R;
-    if ((rows > kGqaSmallRows) != big) continue;
     tiles += (rows + l.tile_rows - 1) / l.tile_rows;
     max_pages = std::max(max_pages, (s.p0 + s.n - 1) / kPageTokens + 1);
   }
@@ -502,13 +483,15 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
     const int rows = s.n * p.R;
     const int t0 = tok0;
     tok0 += s.n;
-    if ((rows > kGqaSmallRows) != big) continue;
+    const int slot = p.expand ? entry : s.slot;  // expanded keys have a table of their own
+    entry += s.n >= p.min_n && s.n <= p.max_n;
+    if (!mine(s)) continue;
     for (int r0 = 0; r0 < rows; r0 += l.tile_rows) {
       const int last = s.p0 + (std::min(r0 + l.tile_rows, rows) - 1) / p.R;
       const int pages = last / kPageTokens + 1;
       const int ns = big ? std::min(want, (pages + kMinSplitPages - 1) / kMinSplitPages) : common;
       for (int k = 0; k < ns; ++k)
-        items.push_back(GqaItem{t0, s.slot, s.p0, r0, rows, (int)((long long)pages * k / ns),
+        items.push_back(GqaItem{t0, slot, s.p0, r0, rows, (int)((long long)pages * k / ns),
                                 (int)((long long)pages * (k + 1) / ns), ns > 1 ? l.parts + k : -1});
       l.n_items += ns;
       if (ns > 1) {
@@ -525,34 +508,86 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
 }
 
 int LayerStack::build_meta(const std::vector<StepSeq>& batch, int M, int n_want, hipStream_t st) {
-  std::vector<std::vector<GqaItem>> items(plans_.size() * 2);
-  std::vector<std::vector<GqaMerge>> merges(plans_.size() * 2);
+  // pieces of the block besides the token rows, in their places
+  std::vector<std::pair<size_t, std::vector<uint8_t>>> pieces;
   size_t at = 0, part_o = 0, part_ml = 0;
   const auto take = [&](size_t bytes) {
     const size_t a = at;
     at += (bytes + 15) / 16 * 16;
     return a;
   };
+  const auto place = [&](const auto& v) {
+    const size_t bytes = v.size() * sizeof(v[0]), a = take(bytes);
+    if (bytes) {
+      const uint8_t* b = reinterpret_cast<const uint8_t*>(v.data());
+      pieces.emplace_back(a, std::vector<uint8_t>(b, b + bytes));
+    }
+    return a;
+  };
   at_tok_ = take((size_t)M * 4);
   at_pos_ = take((size_t)M * 4);
   at_slot_ = take((size_t)M * 4);
+  at_seq0_ = take((size_t)M * 4);
   at_want_ = take((size_t)n_want * 4);
-  for (size_t i = 0; i < plans_.size(); ++i)
+  for (auto& pp : plans_) {
+    Plan& p = *pp;
     for (int b = 0; b < 2; ++b) {
-      Plan& p = plans_[i];
       Launch& l = b ? p.big : p.small;
-      cut(batch, p, b != 0, items[2 * i + b], merges[2 * i + b], l);
-      l.items_at = take(items[2 * i + b].size() * sizeof(GqaItem));
-      l.merges_at = take(merges[2 * i + b].size() * sizeof(GqaMerge));
+      std::vector<GqaItem> items;
+      std::vector<GqaMerge> merges;
+      cut(batch, p, b != 0, items, merges, l);
+      l.items_at = place(items);
+      l.merges_at = place(merges);
       const size_t rows = (size_t)l.parts * p.G * l.tile_rows;
       part_o = std::max(part_o, rows * p.max_pd);
       part_ml = std::max(part_ml, rows * 2);
     }
-  if (part_o > part_o_.n || part_ml > part_ml_.n || at > meta_cap_) {
+    if (p.latent) {
+      std::vector<int32_t> rows;
+      int m = 0;
+      for (const StepSeq& s : batch) {
+        for (int i = 0; i < s.n; ++i)
+          if (s.n >= p.min_n && s.n <= p.max_n) rows.push_back(m + i);
+        m += s.n;
+      }
+      p.n_rows = (int)rows.size();
+      p.rows_at = place(rows);
+    }
+    if (p.expand) {
+      std::vector<int32_t> pos, slot, entry, table;
+      plan_expansion(batch, p, pos, slot, entry, table);
+      p.x_pos = place(pos);
+      p.x_slot = place(slot);
+      p.x_entry = place(entry);
+      p.x_table = place(table);
+      const size_t bytes = (size_t)p.x_pages * kPageTokens * (p.Dp + p.Dvp) * es_;
+      if (bytes > p.pool.n) {
+        LLM_HIP_RET(hipDeviceSynchronize());
+        RET_IF(alloc_zero(p.pool, bytes + bytes / 4));  // (zeros: padding of the rows)
+        LLM_HIP_RET(hipDeviceSynchronize());
+      }
+    }
+  }
+  size_t parts = 0;
+  for (ScanPlan& p : scans_) {
+    std::vector<ScanItem> items, chunks;
+    std::vector<ScanCarry> carry;
+    plan_scan(batch, p, items, chunks, carry);
+    p.items_at = place(items);
+    p.chunks_at = place(chunks);
+    p.carry_at = place(carry);
+    parts = std::max(parts, (size_t)p.parts);
+  }
+  if (part_o > part_o_.n || part_ml > part_ml_.n || at > meta_cap_ ||
+      parts * carry_floats_ > carry_.n) {
     LLM_HIP_RET(hipDeviceSynchronize());
     clear_graphs();
     if (part_o > part_o_.n) RET_IF(part_o_.alloc(part_o * 2));
     if (part_ml > part_ml_.n) RET_IF(part_ml_.alloc(part_ml * 2));
+    if (parts * carry_floats_ > carry_.n) {
+      RET_IF(carry_.alloc(parts * carry_floats_));
+      RET_IF(sum_dt_.alloc(parts * ld_inner_));
+    }
     if (at > meta_cap_) {
       if (h_meta_) LLM_HIP_RET(hipHostFree(h_meta_));
       h_meta_ = nullptr;
@@ -567,24 +602,20 @@ int LayerStack::build_meta(const std::vector<StepSeq>& batch, int M, int n_want,
   int32_t* tok = reinterpret_cast<int32_t*>(h_meta_ + at_tok_);
   int32_t* pos = reinterpret_cast<int32_t*>(h_meta_ + at_pos_);
   int32_t* slot = reinterpret_cast<int32_t*>(h_meta_ + at_slot_);
+  int32_t* seq0 = reinterpret_cast<int32_t*>(h_meta_ + at_seq0_);
   int32_t* want = reinterpret_cast<int32_t*>(h_meta_ + at_want_);
   int m = 0, w = 0;
   for (const StepSeq& s : batch) {
+    const int first = m;
     for (int i = 0; i < s.n_want; ++i) want[w++] = m + s.want[i];
     for (int i = 0; i < s.n; ++i, ++m) {
       tok[m] = s.tokens[i];
       pos[m] = s.p0 + i;
       slot[m] = s.slot;
+      seq0[m] = first;
     }
   }
-  for (size_t i = 0; i < plans_.size(); ++i)
-    for (int b = 0; b < 2; ++b) {
-      const Launch& l = b ? plans_[i].big : plans_[i].small;
-      const auto &it = items[2 * i + b];
-      const auto &me = merges[2 * i + b];
-      if (!it.empty()) std::memcpy(h_meta_ + l.items_at, it.data(), it.size() * sizeof(GqaItem));
-      if (!me.empty()) std::memcpy(h_meta_ + l.merges_at, me.data(), me.size() * sizeof(GqaMerge));
-    }
+  for (const auto& p : pieces) std::memcpy(h_meta_ + p.first, p.second.data(), p.second.size());
   LLM_HIP_RET(hipMemcpyAsync(meta_.p, h_meta_, at, hipMemcpyHostToDevice, st));
   LLM_HIP_RET(hipEventRecord(meta_done_, st));
   return LLM_OK;
@@ -594,7 +625,7 @@ int LayerStack::attention(const Layer& l, const Run& r, int M, hipStream_t st) {
   const AttentionSpec& a = l.s.attn;
   Geometry& g = *geos_[l.geo];
   const KvCache& kv = g.kv;
-  const int32_t* table = kv.d_table + (size_t)r.cache_layer * kv.beams * kv.H * kv.max_tiles;
+  const int32_t* table = table_of(g, r);
   MmArgs p;
   p.A = h_.p;
   p.lda = ldx_;
@@ -624,7 +655,7 @@ int LayerStack::attention(const Layer& l, const Run& r, int M, hipStream_t st) {
   e.page_stride = kv.page_stride();
   LLM_HIP_RET(mm_qkv(dt_, p, e, st));
 
-  const Plan& plan = plans_[l.plan];
+  const Plan& plan = *plans_[l.plan];
   const int ldo = mm_pad(a.heads * a.vdim);
   GqaArgs q;
   q.q = q_.p;
@@ -654,13 +685,17 @@ int LayerStack::attention(const Layer& l, const Run& r, int M, hipStream_t st) {
     LLM_HIP_RET(gqa_attention(dt_, q, c->tile_rows, st));
   }
 
+  return out_product(l, att_.p, ldo, a.heads * a.vdim, M, st);
+}
+
+int LayerStack::out_product(const Layer& l, const void* A, int lda, int K, int M, hipStream_t st) {
   MmArgs o;
-  o.A = att_.p;
-  o.lda = ldo;
+  o.A = A;
+  o.lda = lda;
   o.W = l.o.p;
   o.M = M;
   o.N = cfg_.width;
-  o.K = a.heads * a.vdim;
+  o.K = K;
   o.w_nt = w_nt_;
   o.C = y_.p;
   o.ldc = ldx_;
@@ -668,7 +703,29 @@ int LayerStack::attention(const Layer& l, const Run& r, int M, hipStream_t st) {
   return LLM_OK;
 }
 
-int LayerStack::mlp(const Layer& l, int M, hipStream_t st) {
+int LayerStack::ffn(const Layer& l, int M, hipStream_t st) {
+  MmArgs a;
+  a.A = h_.p;
+  a.lda = ldx_;
+  a.W = l.ffn_in.p;
+  a.M = M;
+  a.N = 2 * l.s.ffn.ff;
+  a.K = cfg_.width;
+  a.w_nt = w_nt_;
+  const int ld = mm_pad(l.s.ffn.ff);
+  LLM_HIP_RET(mm_glu(dt_, a, l.s.ffn.glu, act_.p, ld, st));
+  a.A = act_.p;
+  a.lda = ld;
+  a.W = l.ffn_out.p;
+  a.N = cfg_.width;
+  a.K = l.s.ffn.ff;
+  a.C = y_.p;
+  a.ldc = ldx_;
+  LLM_HIP_RET(mm(dt_, a, st));
+  return LLM_OK;
+}
+
+int LayerStack::moe(const Layer& l, int M, hipStream_t st) {
   const MoeSpec& m = l.s.moe;
   MmArgs z;
   z.A = h_.p;
@@ -737,38 +794,61 @@ int LayerStack::enqueue(int M, int n_want, float* logits, hipStream_t st) {
     n.M = n.M_y = M;
     n.eps = cfg_.eps;
     n.emb = emb_.p;
+    n.emb_scale = cfg_.embedding_scale;
     n.tok = meta<int32_t>(at_tok_);
     n.ldh = ldx_;
     n.h = h_.p;
+    n.streams = cfg_.streams;
   };
-  const auto post = [&](const float* w, int parts, bool shared) {
+  const auto leave = [&](const DevBuf<float>& post, const DevBuf<float>& scale, const Hyper& hc,
+                         int parts, bool shared) {
     fresh();
-    n.w_post = w;
+    n.w_post = post.p;
+    n.y_scale = scale.p;
+    n.hc_mix = hc.mix.p;
+    n.hc_out = hc.out.p;
     n.y = y_.p;
     n.ldy = ldx_;
     n.parts = parts;
     n.shared = shared;
+  };
+  const auto enter = [&](const DevBuf<float>& norm, const Hyper& hc) {
+    n.w_pre = norm.p;
+    n.hc_in = hc.in.p;
+    return rms_norm_step(dt_, n, st);
   };
   fresh();
   n.embed = 1;
   for (size_t i = 0; i < runs_.size(); ++i) {
     const Run& r = runs_[i];
     const Layer& l = *layers_[r.layer];
-    if (r.add_embed) n.embed = 2;
-    n.w_pre = l.norm1.p;
-    LLM_HIP_RET(rms_norm_step(dt_, n, st));
-    RET_IF(attention(l, r, M, st));
-    post(l.norm1b.p, 1, false);
+    if (r.again && cfg_.loop_adds_embedding) n.embed = 2;
+    LLM_HIP_RET(enter(l.norm1, l.hc1));
+    switch (l.s.mixer) {
+      case Mixer::kAttention: RET_IF(attention(l, r, M, st)); break;
+      case Mixer::kLatent: RET_IF(latent(l, r, M, st)); break;
+      case Mixer::kMamba: RET_IF(mamba(l, r, M, st)); break;
+    }
+    leave(l.norm1b, l.ls1, l.hc1, 1, false);
     if (l.s.has_mlp) {
-      n.w_pre = l.norm2.p;
-      LLM_HIP_RET(rms_norm_step(dt_, n, st));
-      RET_IF(mlp(l, M, st));
-      post(l.norm2b.p, l.s.moe.top, l.s.moe.has_shared);
+      LLM_HIP_RET(enter(l.norm2, l.hc2));
+      if (l.s.dense) {
+        RET_IF(ffn(l, M, st));
+        leave(l.norm2b, l.ls2, l.hc2, 1, false);
+      } else {
+        RET_IF(moe(l, M, st));
+        leave(l.norm2b, l.ls2, l.hc2, l.s.moe.top, l.s.moe.has_shared);
+      }
     }
     if (tap_) {
+      const float* rows = x_.p;
+      if (cfg_.streams > 0) {  // the sum of the streams
+        if (tap_rows_.n < (size_t)M * ldx_) RET_IF(tap_rows_.alloc((size_t)M * ldx_));
+        rows = n.u = tap_rows_.p;
+      }
       LLM_HIP_RET(rms_norm_step(dt_, n, st));
       fresh();
-      LLM_HIP_RET(hipMemcpy2DAsync(tap_ + i * (size_t)M * cfg_.width, (size_t)cfg_.width * 4, x_.p,
+      LLM_HIP_RET(hipMemcpy2DAsync(tap_ + i * (size_t)M * cfg_.width, (size_t)cfg_.width * 4, rows,
                                    (size_t)ldx_ * 4, (size_t)cfg_.width * 4, M,
                                    hipMemcpyDeviceToHost, st));
     }
@@ -788,6 +868,7 @@ int LayerStack::enqueue(int M, int n_want, float* logits, hipStream_t st) {
   a.w_nt = w_nt_;
   a.C = logits;
   a.ldc = cfg_.vocab;
+  a.softcap = cfg_.logit_softcap;
   LLM_HIP_RET(mm(dt_, a, st));
   return LLM_OK;
 }
@@ -795,6 +876,7 @@ int LayerStack::enqueue(int M, int n_want, float* logits, hipStream_t st) {
 int LayerStack::forward(const std::vector<StepSeq>& batch, float* logits, hipStream_t st) {
   int M = 0, n_want = 0;
   bool decode = true;
+  single_ = true;
   std::vector<char> seen(opt_.max_seqs, 0);
   for (const StepSeq& s : batch) {
     LLM_REQUIRE(s.slot >= 0 && s.slot < opt_.max_seqs && !seen[s.slot], "step: bad or repeated slot");
@@ -807,6 +889,7 @@ int LayerStack::forward(const std::vector<StepSeq>& batch, float* logits, hipStr
       LLM_REQUIRE(s.want && s.want[i] >= 0 && s.want[i] < s.n, "step: wanted place out of range");
     M += s.n;
     n_want += s.n_want;
+    single_ = single_ && s.n == 1;
     decode = decode && s.n == 1 && s.n_want == 1;
   }
   LLM_REQUIRE(M >= 1 && M <= cap_ && n_want <= M, "step: too many tokens");
@@ -824,8 +907,8 @@ int LayerStack::forward(const std::vector<StepSeq>& batch, float* logits, hipStr
   if (!use_graph_ || !decode || tap_) return enqueue(M, n_want, logits, st);
 
   std::vector<long long> key{M, (long long)reinterpret_cast<uintptr_t>(logits)};
-  for (const Plan& p : plans_)
-    for (const Launch* l : {&p.small, &p.big})
+  for (const auto& p : plans_)
+    for (const Launch* l : {&p->small, &p->big})
       key.insert(key.end(), {l->n_items, l->n_merges});
   auto it = graphs_.find(key);
   if (it == graphs_.end()) {  // first of its shape: run it, capture the next
@@ -863,8 +946,6 @@ int LayerStack::release(int slot) {
   }
   return LLM_OK;
 }
-
-}  // namespace
 
 int make_layer_stack(const LayerStackConfig& cfg, const std::string& dir, const ModelOptions& opt,
                      std::unique_ptr<StepModel>* out) {

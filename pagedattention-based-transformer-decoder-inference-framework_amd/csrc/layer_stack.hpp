@@ -1,6 +1,7 @@
 // Decoder-only models given as a list of layers (csrc/layer_stack.cpp): every
 // layer names its mixer and its feed-forward with sizes of their own, a run of
-// layers may repeat with the same weights, norms stand before and after each
+// layers may repeat with the same weights, norms stand before (and after) each
+// sublayer, and the residual is one stream or several that are mixed around each
 // sublayer.  A model family reads its config.json into LayerStackConfig.
 #pragma once
 
@@ -35,6 +36,20 @@ struct AttentionSpec {
   bool sink = false;  // a learned term in each head's softmax denominator
 };
 
+// Keys and values are products of one normed latent per token; a rotated key part
+// is shared by the heads.  The cache holds the latent and that part.
+struct LatentSpec {
+  int heads = 0, dim = 0, rot_dim = 0, vdim = 0, rank = 0;
+  RopeSpec rope;  // dims = rot_dim, partners side by side
+  float scale = 1.f;
+  bool sink = false;
+};
+
+// Selective scan behind a short causal convolution.
+struct MambaSpec {
+  int inner = 0, state = 0, dt_rank = 0, taps = 0;
+};
+
 struct ExpertSpec {
   int ff = 0;
   GluParams glu;
@@ -47,9 +62,16 @@ struct MoeSpec {
   ExpertSpec shared;
 };
 
+enum class Mixer { kAttention, kLatent, kMamba };
+
 struct LayerSpec {
+  Mixer mixer = Mixer::kAttention;
   AttentionSpec attn;
+  LatentSpec latent;
+  MambaSpec mamba;
   bool has_mlp = false;
+  bool dense = false;  // the feed-forward is `ffn`, otherwise `moe`
+  ExpertSpec ffn;
   MoeSpec moe;
 };
 
@@ -57,9 +79,15 @@ struct LayerStackConfig {
   int vocab = 0, width = 0;
   float eps = 1e-5f;
   std::vector<LayerSpec> layers;
-  // layers [loop_start, loop_stop) are passed through loop_times times; a repeated
-  // pass starts with the tokens' embeddings added to the residual once more
+  // layers [loop_start, loop_stop) are passed through loop_times times
   int loop_start = 0, loop_stop = 0, loop_times = 1;
+  // a repeated pass starts with the tokens' embeddings added to the residual
+  bool loop_adds_embedding = false;
+  float embedding_scale = 1.f;
+  bool post_norm = false;    // sublayer outputs are normed (norm1b, norm2b)
+  bool layer_scale = false;  // and multiplied element by element (ls1, ls2)
+  int streams = 0;           // residual streams mixed by hc1.*, hc2.* (0: one, plain sums)
+  float logit_softcap = 0.f;  // 0: none
 };
 
 // Checks the configuration, reads the weights of dir/model.safetensors (tensor

@@ -1,417 +1,10 @@
-// Matrix products of the layer-stack models on gfx950 MFMA.
-//
-//   bf16: v_mfma_f32_16x16x32_bf16      fp32: v_mfma_f32_16x16x4_f32
-//
-// Two kernels.  Decode rows stream: a block owns 16 MT rows x 16 NT columns, its
-// 8 waves split K and load A (row-major rows, 64 bytes per row and k-step) and W
-// (packed 1 KiB fragments) straight into registers, so every weight byte of the
-// product is in flight at once.  Prompt rows go through LDS in 128 x 128 (or 64 x
-// 128) blocks, both operands loaded from memory into LDS in fragment order.
-// Grouped rows take either form; a tile list (built by the routing kernel) names
-// the group and rows of each row of the grid.
-// A and W share the k order inside a fragment, so the sum is exact whatever the
-// hardware's own order; C: column = lane & 15, row = 4 (lane >> 4) + reg.
-//
-// Epilogues work on column pairs (2i, 2i + 1), which sit in neighbouring lanes:
-// rotation partners and (gate, up) pairs are packed side by side, so a pair is
-// one DPP move away and no product needs a second launch to finish it.
-#include "common.hpp"
-#include "mm.hpp"
-
-#include <algorithm>
+// Matrix products of the layer-stack models: packing, plain products, the
+// grouped-query projections and the grouped (expert) products.  The kernels are
+// in mm_impl.hpp; mm_mix.hip has the epilogues of the other mixers.
+#include "mm_impl.hpp"
 
 namespace llm {
 namespace {
-
-typedef __bf16 bf16x8 __attribute__((ext_vector_type(8)));
-
-enum Epi { kStore, kQkv, kGroupIn, kGroupOut };
-
-template <typename T>
-struct Kind;
-template <>
-struct Kind<__bf16> {
-  static constexpr bool BF16 = true;
-  static __device__ __forceinline__ f32x4 mma(u32x4 a, u32x4 b, f32x4 c) {
-    return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a),
-                                                   __builtin_bit_cast(bf16x8, b), c, 0, 0, 0);
-  }
-};
-template <>
-struct Kind<float> {
-  static constexpr bool BF16 = false;
-  static __device__ __forceinline__ f32x4 mma(u32x4 a, u32x4 b, f32x4 c) {
-    const f32x4 x = __builtin_bit_cast(f32x4, a), y = __builtin_bit_cast(f32x4, b);
-#pragma unroll
-    for (int j = 0; j < 4; ++j) c = __builtin_amdgcn_mfma_f32_16x16x4f32(x[j], y[j], c, 0, 0, 0);
-    return c;
-  }
-};
-
-struct KernelArgs {
-  MmArgs a;
-  int KS;
-  MmQkv q;
-  MmGrouped g;
-};
-
-__device__ __forceinline__ float glu(float gate, float up, const GluParams& p) {
-  const float g = fminf(gate, p.limit);
-  const float u = fminf(fmaxf(up, -p.limit), p.limit);
-  return g / (1.f + expf(-p.alpha * g)) * (u + p.up_bias);
-}
-
-template <typename T>
-__device__ __forceinline__ void put_pair(T* p, float v0, float v1) {
-  typedef T pair_t __attribute__((ext_vector_type(2)));
-  pair_t v;
-  v[0] = (T)v0;
-  v[1] = (T)v1;
-  *reinterpret_cast<pair_t*>(p) = v;
-}
-
-// What a block of rows and columns works on: set once from the launch arguments
-// or the tile list.
-template <typename T>
-struct Block {
-  const T* A = nullptr;
-  const char* W = nullptr;
-  int lda = 0, M = 0, N = 0, KS = 0, m0 = 0;
-  bool shared = false;
-  GluParams glu;
-};
-
-template <typename T, int EPI>
-__device__ __forceinline__ Block<T> block_of(const KernelArgs& p, int row_blocks) {
-  Block<T> b;
-  if constexpr (EPI == kGroupIn || EPI == kGroupOut) {
-    const MmTile t = p.g.tiles[blockIdx.y];
-    const MmGroup g = p.g.groups[t.group];
-    b.shared = t.group >= p.g.n_routed;
-    b.m0 = t.row0;
-    b.M = t.row0 + t.rows;
-    if constexpr (EPI == kGroupIn) {
-      b.A = static_cast<const T*>(p.g.h);
-      b.lda = p.g.ldh;
-      b.W = static_cast<const char*>(g.w_in);
-      b.N = g.n_in;
-      b.KS = g.ks_in;
-      b.glu = g.glu;
-    } else {
-      b.A = static_cast<const T*>(b.shared ? p.g.act_shared : p.g.act);
-      b.lda = b.shared ? p.g.lds : p.g.lda;
-      b.W = static_cast<const char*>(g.w_out);
-      b.N = g.n_out;
-      b.KS = g.ks_out;
-    }
-  } else {
-    b.A = static_cast<const T*>(p.a.A);
-    b.W = static_cast<const char*>(p.a.W);
-    b.lda = p.a.lda;
-    b.M = p.a.M;
-    b.N = p.a.N;
-    b.KS = p.KS;
-    b.m0 = (int)blockIdx.y * row_blocks;
-  }
-  return b;
-}
-
-// This lane's 16 bytes of the first k-step of row m's fragments.
-template <typename T, int EPI>
-__device__ __forceinline__ const char* a_lane(const KernelArgs& p, const Block<T>& b, int m) {
-  m = min(m, b.M - 1);
-  if constexpr (EPI == kGroupIn) {
-    if (!b.shared) m = p.g.perm[m] / p.g.top;
-  }
-  return reinterpret_cast<const char*>(b.A + (size_t)m * b.lda) + 16 * (lane_id() >> 4);
-}
-
-// Where the column pair (n, n + 1) of row m goes, and what it still needs: found
-// before the sums are there, so the loads behind it (position, slot, page,
-// angle, assignment) overlap the weight stream.
-template <typename T, int EPI>
-struct Target {
-  void* p0 = nullptr;  // NULL: nothing to write
-  void* p1 = nullptr;  // the second column's place where it is not next to the first
-  float cs = 1.f, sn = 0.f;  // rotation; kGroupOut: cs is the weight
-
-  __device__ __forceinline__ void find(const KernelArgs& p, const Block<T>& b, int m, int n) {
-    if (m >= b.M || n >= b.N) return;
-    if constexpr (EPI == kStore) {
-      float* d = p.a.C + (size_t)m * p.a.ldc + n;
-      p0 = d;
-      p1 = n + 1 < b.N ? d + 1 : nullptr;
-    } else if constexpr (EPI == kGroupIn) {
-      T* d = static_cast<T*>(b.shared ? p.g.act_shared : p.g.act);
-      p0 = d + (size_t)m * (b.shared ? p.g.lds : p.g.lda) + (n >> 1);
-    } else if constexpr (EPI == kGroupOut) {
-      const int row = b.shared ? p.g.M * p.g.top + m : p.g.perm[m];
-      if (!b.shared) cs = p.g.weight[row];
-      float* d = p.g.out + (size_t)row * p.g.ldo + n;
-      p0 = d;
-      p1 = n + 1 < b.N ? d + 1 : nullptr;
-    } else {
-      const MmQkv& e = p.q;
-      const int nq = e.H * e.D, nk = e.G * e.D;
-      if (n < nq) {
-        const int head = n / e.D, d = n - head * e.D;
-        turn(e, m, d);
-        p0 = static_cast<T*>(e.q) + ((size_t)m * e.H + head) * e.Dp + d;
-        return;
-      }
-      const int pos = e.pos[m], tile = pos / kPageTokens, at = pos % kPageTokens;
-      if (tile >= e.max_tiles) return;
-      const int32_t* table = e.table + (size_t)e.slot[m] * e.G * e.max_tiles + tile;
-      if (n < nq + nk) {
-        const int head = (n - nq) / e.D, d = n - nq - head * e.D;
-        turn(e, m, d);
-        char* page = page_of(e, e.k_pool, table[(size_t)head * e.max_tiles]);
-        if (page) p0 = reinterpret_cast<T*>(page) + (size_t)at * e.Dp + d;
-        return;
-      }
-      const int v = n - nq - nk, slot = v_page_slot(at, Kind<T>::BF16);
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const int head = (v + j) / e.Dv, d = v + j - head * e.Dv;
-        if (head >= e.G) break;  // the second half of the last pair
-        char* page = page_of(e, e.v_pool, table[(size_t)head * e.max_tiles]);
-        if (page) (j ? p1 : p0) = reinterpret_cast<T*>(page) + (size_t)d * kPageTokens + slot;
-      }
-    }
-  }
-
-  __device__ __forceinline__ void put(const KernelArgs& p, const Block<T>& b, int n, float v0,
-                                      float v1) const {
-    if constexpr (EPI == kStore || EPI == kGroupOut) {
-      if (p0) *static_cast<float*>(p0) = EPI == kGroupOut ? cs * v0 : v0;
-      if (p1) *static_cast<float*>(p1) = EPI == kGroupOut ? cs * v1 : v1;
-    } else if constexpr (EPI == kGroupIn) {
-      if (p0) *static_cast<T*>(p0) = (T)glu(v0, v1, b.glu);
-    } else {
-      if (n < (p.q.H + p.q.G) * p.q.D) {
-        if (p0) put_pair(static_cast<T*>(p0), v0 * cs - v1 * sn, v1 * cs + v0 * sn);
-      } else {
-        if (p0) *static_cast<T*>(p0) = (T)v0;
-        if (p1) *static_cast<T*>(p1) = (T)v1;
-      }
-    }
-  }
-
- private:
-  __device__ __forceinline__ void turn(const MmQkv& e, int m, int d) {
-    if (d >= e.rot) return;
-    const float2 t = e.turn[(size_t)m * (e.rot >> 1) + (d >> 1)];
-    cs = t.x;
-    sn = t.y;
-  }
-  static __device__ __forceinline__ char* page_of(const MmQkv& e, void* pool, int page) {
-    return page >= 0 && page < e.num_pages ? static_cast<char*>(pool) + (size_t)page * e.page_stride
-                                           : nullptr;
-  }
-};
-
-// One 16 x 16 tile of finished sums (rows m0.., columns n0..) -> the epilogue,
-// a column pair per lane.  Every lane of the wave takes part.
-template <typename T, int EPI>
-__device__ __forceinline__ void emit_tile(const KernelArgs& p, const Block<T>& b, f32x4 c, int m0,
-                                          int n0) {
-  const int lane = lane_id();
-  f32x4 o;
-#pragma unroll
-  for (int r = 0; r < 4; ++r) o[r] = mov_dpp<0xB1>(c[r]);  // the neighbouring column
-  const bool odd = lane & 1;
-  const int n = n0 + (lane & 14);
-#pragma unroll
-  for (int r = 0; r < 2; ++r) {
-    Target<T, EPI> t;
-    t.find(p, b, m0 + 4 * (lane >> 4) + (odd ? 2 : 0) + r, n);
-    t.put(p, b, n, odd ? o[2 + r] : c[r], odd ? c[2 + r] : o[r]);
-  }
-}
-
-// Decode rows (and short grouped tiles): a block owns 16 MT rows x 16 NT columns
-// and its WK waves split K, adding through LDS in a fixed order.
-template <typename T, int EPI, int MT, int NT, int WK>
-__global__ __launch_bounds__(64 * WK, MT * NT == 1 ? 4 : 2) void mm_stream_kernel(KernelArgs p) {
-  if constexpr (EPI == kGroupIn || EPI == kGroupOut)
-    if ((int)blockIdx.y >= *p.g.n_tiles) return;
-  constexpr int U = MT * NT >= 4 ? 2 : 4;  // k-steps per load batch
-  const int lane = lane_id();
-  const int w = wave_id_uniform();
-  const Block<T> b = block_of<T, EPI>(p, 16 * MT);
-  const int ntiles = (b.N + 15) >> 4;
-  const int nt0 = (int)blockIdx.x * NT;
-  if (nt0 >= ntiles) return;  // (groups differ in width)
-
-  const char* ap[MT];
-#pragma unroll
-  for (int i = 0; i < MT; ++i) ap[i] = a_lane<T, EPI>(p, b, b.m0 + 16 * i + (lane & 15));
-  const char* bp[NT];
-#pragma unroll
-  for (int j = 0; j < NT; ++j)
-    bp[j] = b.W + (size_t)min(nt0 + j, ntiles - 1) * b.KS * 1024 + lane * 16;
-
-  f32x4 acc[MT][NT];
-#pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-
-  // Neighbouring blocks start at different k ranges, so they do not all pull
-  // the same A lines at once.
-  const int wr = (w + (int)blockIdx.x) % WK;
-  const int ks0 = wr * b.KS / WK, ks1 = (wr + 1) * b.KS / WK;
-  struct Batch {
-    u32x4 a[U][MT], b[U][NT];
-  };
-  const bool nt_load = p.a.w_nt;
-  auto load = [&](Batch& x, int ks) {
-#pragma unroll
-    for (int u = 0; u < U; ++u) {
-      const int k = ks + u;
-      if (k < ks1) {
-#pragma unroll
-        for (int j = 0; j < NT; ++j) {
-          const u32x4* src = reinterpret_cast<const u32x4*>(bp[j] + (size_t)k * 1024);
-          x.b[u][j] = nt_load ? __builtin_nontemporal_load(src) : *src;
-        }
-#pragma unroll
-        for (int i = 0; i < MT; ++i)
-          x.a[u][i] = *reinterpret_cast<const u32x4*>(ap[i] + (size_t)k * 64);
-      } else {
-#pragma unroll
-        for (int j = 0; j < NT; ++j) x.b[u][j] = u32x4{0u, 0u, 0u, 0u};
-#pragma unroll
-        for (int i = 0; i < MT; ++i) x.a[u][i] = u32x4{0u, 0u, 0u, 0u};
-      }
-    }
-  };
-  auto mul = [&](const Batch& x) {
-#pragma unroll
-    for (int u = 0; u < U; ++u)
-#pragma unroll
-      for (int i = 0; i < MT; ++i)
-#pragma unroll
-        for (int j = 0; j < NT; ++j) acc[i][j] = Kind<T>::mma(x.a[u][i], x.b[u][j], acc[i][j]);
-  };
-  // thread t finishes column pairs t, t + THREADS, ...: 8 pairs a row, 128 a tile
-  constexpr int PAIRS = MT * NT * 128, THREADS = 64 * WK, EPT = (PAIRS + THREADS - 1) / THREADS;
-  __shared__ float red[WK][MT * NT][4][64];
-  Target<T, EPI> target[EPT];
-  Batch x, y;
-  if (ks0 < ks1) load(x, ks0);
-#pragma unroll
-  for (int e = 0; e < EPT; ++e) {
-    const int pr = threadIdx.x + e * THREADS, t = pr >> 7;
-    if (pr < PAIRS)
-      target[e].find(p, b, b.m0 + 16 * (t / NT) + ((pr >> 3) & 15),
-                     (nt0 + t % NT) * 16 + (pr & 7) * 2);
-  }
-  if (ks0 < ks1) {
-    for (int ks = ks0;;) {
-      if (ks + U < ks1) load(y, ks + U);
-      mul(x);
-      ks += U;
-      if (ks >= ks1) break;
-      if (ks + U < ks1) load(x, ks + U);
-      mul(y);
-      ks += U;
-      if (ks >= ks1) break;
-    }
-  }
-
-#pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) red[wr][i * NT + j][r][lane] = acc[i][j][r];
-  __syncthreads();
-#pragma unroll
-  for (int e = 0; e < EPT; ++e) {
-    const int pr = threadIdx.x + e * THREADS;
-    if (pr >= PAIRS) break;
-    const int t = pr >> 7, row = (pr >> 3) & 15, col = (pr & 7) * 2;
-    float2 s = {0.f, 0.f};
-#pragma unroll
-    for (int k = 0; k < WK; ++k) {
-      const float2 v = *reinterpret_cast<const float2*>(&red[k][t][row & 3][(row >> 2) * 16 + col]);
-      s.x += v.x;
-      s.y += v.y;
-    }
-    target[e].put(p, b, (nt0 + t % NT) * 16 + col, s.x, s.y);
-  }
-}
-
-// Prompt rows: a block of 16 MB rows x 128 columns, 4 waves as WM x (4 / WM).
-// Fragments go from memory straight into LDS (A gathered row by row, W linear),
-// two k-steps per stage, the next stage in flight while one is multiplied.
-template <typename T, int EPI, int MB, int WM>
-__global__ __launch_bounds__(256, 2) void mm_block_kernel(KernelArgs p) {
-  if constexpr (EPI == kGroupIn || EPI == kGroupOut)
-    if ((int)blockIdx.y >= *p.g.n_tiles) return;
-  constexpr int NB = 8, WN = 4 / WM, MT = MB / WM, NT = NB / WN;
-  constexpr int AW = MB / 4, BW = NB / 4;  // row / column tiles a wave loads
-  __shared__ u32x4 sa[2][2][MB][64];       // [stage][k-step][tile][lane]
-  __shared__ u32x4 sb[2][2][NB][64];
-  const int lane = lane_id();
-  const int w = wave_id_uniform();
-  const Block<T> b = block_of<T, EPI>(p, 16 * MB);
-  const int ntiles = (b.N + 15) >> 4;
-  const int nt0 = (int)blockIdx.x * NB;
-  if (nt0 >= ntiles) return;
-
-  const char* ap[AW];
-#pragma unroll
-  for (int i = 0; i < AW; ++i)
-    ap[i] = a_lane<T, EPI>(p, b, b.m0 + 16 * (w * AW + i) + (lane & 15));
-  const char* bp[BW];
-#pragma unroll
-  for (int j = 0; j < BW; ++j)
-    bp[j] = b.W + (size_t)min(nt0 + w * BW + j, ntiles - 1) * b.KS * 1024 + lane * 16;
-  auto issue = [&](int st, int ks) {
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      if (ks + u >= b.KS) break;
-#pragma unroll
-      for (int i = 0; i < AW; ++i) load_to_lds(ap[i] + (size_t)(ks + u) * 64, sa[st][u][w * AW + i]);
-#pragma unroll
-      for (int j = 0; j < BW; ++j)
-        load_to_lds(bp[j] + (size_t)(ks + u) * 1024, sb[st][u][w * BW + j]);
-    }
-  };
-  const int wm = w / WN, wn = w % WN;
-  f32x4 acc[MT][NT];
-#pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  auto mul = [&](int st, int u) {
-    u32x4 a[MT], c[NT];
-#pragma unroll
-    for (int i = 0; i < MT; ++i) a[i] = sa[st][u][wm * MT + i][lane];
-#pragma unroll
-    for (int j = 0; j < NT; ++j) c[j] = sb[st][u][wn * NT + j][lane];
-#pragma unroll
-    for (int i = 0; i < MT; ++i)
-#pragma unroll
-      for (int j = 0; j < NT; ++j) acc[i][j] = Kind<T>::mma(a[i], c[j], acc[i][j]);
-  };
-  issue(0, 0);
-  int st = 0;
-  for (int ks = 0; ks < b.KS; ks += 2, st ^= 1) {
-    wait_lds_loads();
-    __syncthreads();  // stage st has landed, stage st ^ 1 is read out
-    if (ks + 2 < b.KS) issue(st ^ 1, ks + 2);
-    mul(st, 0);
-    if (ks + 1 < b.KS) mul(st, 1);
-  }
-#pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j)
-      emit_tile<T, EPI>(p, b, acc[i][j], b.m0 + 16 * (wm * MT + i), (nt0 + wn * NT + j) * 16);
-}
 
 template <typename T>
 __global__ void mm_pack_kernel(const uint16_t* __restrict__ src, const int32_t* __restrict__ map,
@@ -437,53 +30,6 @@ __global__ void mm_pack_kernel(const uint16_t* __restrict__ src, const int32_t* 
   u32x4 o;
   __builtin_memcpy(&o, v, 16);
   dst[idx] = o;
-}
-
-template <typename T, int EPI, int MT, int NT, int WK = 8>
-hipError_t stream(const KernelArgs& p, int row_blocks, int N, hipStream_t st) {
-  const dim3 grid(((N + 15) / 16 + NT - 1) / NT, row_blocks);
-  hipLaunchKernelGGL((mm_stream_kernel<T, EPI, MT, NT, WK>), grid, dim3(64 * WK), 0, st, p);
-  return hipGetLastError();
-}
-
-template <typename T, int EPI, int MB, int WM>
-hipError_t blocks(const KernelArgs& p, int row_blocks, int N, hipStream_t st) {
-  const dim3 grid((N + 127) / 128, row_blocks);
-  hipLaunchKernelGGL((mm_block_kernel<T, EPI, MB, WM>), grid, dim3(256), 0, st, p);
-  return hipGetLastError();
-}
-
-template <typename T, int EPI>
-hipError_t launch(const KernelArgs& p, hipStream_t st) {
-  const int M = p.a.M, N = p.a.N;
-  const int ntiles = (N + 15) / 16;
-  // rows in blocks of 16 (the weights of the later blocks come from L2): 64 x
-  // 2560 x 2048 10.8 us, against 12.8 in blocks of 32 and 13.8 in one of 64
-  const int b16 = (M + 15) / 16;
-  if (M <= 16) return stream<T, EPI, 1, 1>(p, 1, N, st);
-  // two column tiles per block once that still fills the chip
-  if (M <= 64 && ntiles >= 512)
-    return M <= 32 ? stream<T, EPI, 2, 2>(p, 1, N, st) : stream<T, EPI, 4, 2>(p, 1, N, st);
-  if (M <= 64)
-    return ntiles * b16 < 256 ? stream<T, EPI, 1, 1>(p, b16, N, st)
-                              : stream<T, EPI, 1, 2>(p, b16, N, st);
-  // prompt rows: blocks once there are enough of them, else 32-row streams
-  const int n128 = (N + 127) / 128;
-  if ((M + 127) / 128 * n128 >= 256) return blocks<T, EPI, 8, 2>(p, (M + 127) / 128, N, st);
-  if ((M + 63) / 64 * n128 >= 128) return blocks<T, EPI, 4, 1>(p, (M + 63) / 64, N, st);
-  return stream<T, EPI, 2, 1>(p, (M + 31) / 32, N, st);
-}
-
-template <typename T, int EPI>
-hipError_t launch_grouped(const MmGrouped& g, int w_nt, hipStream_t st) {
-  KernelArgs p{};
-  p.g = g;
-  p.a.w_nt = w_nt;
-  if (g.tile_rows == 128) return blocks<T, EPI, 8, 2>(p, g.max_tiles, g.max_n, st);
-  if (g.tile_rows == 64) return blocks<T, EPI, 4, 1>(p, g.max_tiles, g.max_n, st);
-  // few k-steps per wave are not worth eight of them
-  return g.min_ks >= 16 ? stream<T, EPI, 1, 1>(p, g.max_tiles, g.max_n, st)
-                        : stream<T, EPI, 1, 1, 4>(p, g.max_tiles, g.max_n, st);
 }
 
 }  // namespace

@@ -100,9 +100,86 @@ struct MmArgs {
   int w_nt = 0;             // weights streamed once per step (not kept in cache)
   float* C = nullptr;       // [M][ldc]
   int ldc = 0;
+  float softcap = 0.f;      // C = softcap tanh(C / softcap) when set
+};
+
+// Columns [0, n_t) go to `t` in the element type, the others to `f` in fp32
+// (from its column 0).  n_t and the row lengths are even; an odd N may write its
+// padding column.
+struct MmSplit {
+  void* t = nullptr;
+  int ldt = 0, n_t = 0;
+  float* f = nullptr;
+  int ldf = 0;
+};
+
+// The input product of a layer with a short causal convolution, for rows that
+// are one token each: columns [0, channels) pass the convolution of the row's
+// slot and silu into `x`, and shift its history; columns from `gate` on go to z.
+constexpr int kMmConvTaps = 4;  // most taps this epilogue takes
+struct MmConv {
+  int channels = 0, gate = 0, taps = 0;
+  const int32_t* pos = nullptr;   // [M]
+  const int32_t* slot = nullptr;  // [M]
+  const float* w = nullptr;       // [taps][ldw], the last tap is the current token's
+  const float* bias = nullptr;    // [ldw]
+  int ldw = 0;
+  void* history = nullptr;        // [slots][taps - 1][ldw], oldest first
+  void* x = nullptr;
+  int ldx = 0;
+  void* z = nullptr;
+  int ldz = 0;
+};
+
+// Projections of a latent-attention layer: H heads of D + rot query columns (D
+// and rot even; partners of a rotation are columns 2i and 2i + 1), then the
+// latent and the shared key part in fp32 (not turned).  Queries go to `q`; their
+// turned part also behind the latent part of `q_lat`.
+struct MmLatent {
+  const float2* turn = nullptr;   // [M][rot / 2]
+  int H = 0, D = 0, rot = 0;
+  void* q = nullptr;              // [M][H][ldq]: D, then rot
+  int ldq = 0;
+  void* q_lat = nullptr;          // [M][H][ld_lat], turned part at `lat_rot`
+  int ld_lat = 0, lat_rot = 0;
+  float* down = nullptr;          // [M][ldd]
+  int ldd = 0;
+};
+
+// One product per head: A and C move by a_head / c_head elements, W by w_head
+// bytes.  With `rows` only these rows of A and C take part (M: their number).
+struct MmHeads {
+  int heads = 1;
+  size_t a_head = 0, w_head = 0;
+  void* C = nullptr;
+  int ldc = 0, c_head = 0;
+  const int32_t* rows = nullptr;
+};
+
+// Rows of A taken from cache pages: row m is token pos[m] of page-table row
+// slot[m] (MmArgs::A and lda unused).
+struct MmPageRows {
+  const int32_t* pos = nullptr;
+  const int32_t* slot = nullptr;
+  const int32_t* table = nullptr;  // [slots][max_tiles]
+  int max_tiles = 0, num_pages = 0;
+  const void* pool = nullptr;      // page: [kPageTokens][row]
+  size_t page_stride = 0;          // bytes
+  int row = 0;                     // elements
 };
 
 hipError_t mm(int dtype, const MmArgs& a, hipStream_t st);
+hipError_t mm_split(int dtype, const MmArgs& a, const MmSplit& e, hipStream_t st);
+// W holds gate and up rows interleaved (N = 2 ff); act [M][ld] = glu
+hipError_t mm_glu(int dtype, const MmArgs& a, const GluParams& p, void* act, int ld, hipStream_t st);
+// C = softplus(A . W^T + bias), bias padded to an even length
+hipError_t mm_softplus(int dtype, const MmArgs& a, const float* bias, hipStream_t st);
+hipError_t mm_conv(int dtype, const MmArgs& a, const MmConv& e, hipStream_t st);
+hipError_t mm_latent(int dtype, const MmArgs& a, const MmLatent& e, hipStream_t st);
+hipError_t mm_heads(int dtype, const MmArgs& a, const MmHeads& e, hipStream_t st);
+// keys and values (no queries, e.H = 0, not turned) of the rows of cache pages,
+// into the pages of e
+hipError_t mm_expand(int dtype, const MmArgs& a, const MmPageRows& r, const MmQkv& e, hipStream_t st);
 hipError_t mm_qkv(int dtype, const MmArgs& a, const MmQkv& e, hipStream_t st);
 // act = glu(h . w_in^T) of every group's rows
 hipError_t mm_grouped_in(int dtype, const MmGrouped& g, int w_nt, hipStream_t st);

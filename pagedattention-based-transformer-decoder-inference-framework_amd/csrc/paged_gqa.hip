@@ -203,7 +203,8 @@ struct Rows {
         den = l[t] * f + __builtin_amdgcn_exp2f(s2 - m2);
       }
       f /= den;
-      T* dst = static_cast<T*>(a.out) + (size_t)(it.tok0 + tok) * a.ldo + (size_t)head * a.Dv;
+      T* dst = static_cast<T*>(a.out) + (size_t)(it.tok0 + tok) * a.ldo +
+             (size_t)head * (a.ldh ? a.ldh : a.Dv);
 #pragma unroll
       for (int n = 0; n < ND; ++n)
 #pragma unroll
@@ -428,7 +429,7 @@ __global__ __launch_bounds__(64 * kWaves, 2) void gqa_rows_kernel(GqaArgs a) {
 }
 
 // One wave per row of a split tile.
-template <typename T>
+template <typename T, int MAXD>
 __global__ __launch_bounds__(256) void gqa_merge_kernel(GqaArgs a, int TR) {
   const GqaMerge it = a.merges[blockIdx.x];
   const int kvh = blockIdx.y, R = a.H / a.G, lane = lane_id();
@@ -446,29 +447,30 @@ __global__ __launch_bounds__(256) void gqa_merge_kernel(GqaArgs a, int TR) {
     const float wgt = mine ? __builtin_amdgcn_exp2f(st.x - m) : 0.f;
     float den = wave_sum(mine ? st.y * wgt : 0.f);
     if (a.sink) den += __builtin_amdgcn_exp2f(s2 - m);
-    float acc[kGqaMaxDim / 64] = {};
+    float acc[MAXD / 64] = {};
     constexpr int U = 8;  // splits in flight
     for (int k = 0; k < it.nsplit; k += U) {
-      float v[U][kGqaMaxDim / 64];
+      float v[U][MAXD / 64];
 #pragma unroll
       for (int u = 0; u < U; ++u) {
         const int sp = min(k + u, it.nsplit - 1);
         const float* src = a.part_o + (((size_t)(it.part0 + sp) * a.G + kvh) * TR + rr) * pd;
 #pragma unroll
-        for (int j = 0; j < kGqaMaxDim / 64; ++j)
+        for (int j = 0; j < MAXD / 64; ++j)
           if (lane + 64 * j < a.Dv) v[u][j] = src[lane + 64 * j];
       }
 #pragma unroll
       for (int u = 0; u < U; ++u) {
         const float ws = k + u < it.nsplit ? __shfl(wgt, k + u, 64) : 0.f;
 #pragma unroll
-        for (int j = 0; j < kGqaMaxDim / 64; ++j)
+        for (int j = 0; j < MAXD / 64; ++j)
           if (lane + 64 * j < a.Dv) acc[j] += ws * v[u][j];
       }
     }
-    T* dst = static_cast<T*>(a.out) + (size_t)(it.tok0 + tok) * a.ldo + (size_t)head * a.Dv;
+    T* dst = static_cast<T*>(a.out) + (size_t)(it.tok0 + tok) * a.ldo +
+             (size_t)head * (a.ldh ? a.ldh : a.Dv);
 #pragma unroll
-    for (int j = 0; j < kGqaMaxDim / 64; ++j)
+    for (int j = 0; j < MAXD / 64; ++j)
       if (lane + 64 * j < a.Dv) dst[lane + 64 * j] = (T)(acc[j] / den);
   }
 }
@@ -476,8 +478,11 @@ __global__ __launch_bounds__(256) void gqa_merge_kernel(GqaArgs a, int TR) {
 template <typename T>
 hipError_t merge(const GqaArgs& a, int tile_rows, hipStream_t st) {
   if (a.n_merges <= 0) return hipSuccess;
-  hipLaunchKernelGGL(gqa_merge_kernel<T>, dim3(a.n_merges, a.G, std::min(tile_rows / 4, 8)),
-                     dim3(256), 0, st, a, tile_rows);
+  const dim3 grid(a.n_merges, a.G, std::min(tile_rows / 4, 8));
+  if (a.Dv <= kGqaMaxDim)
+    hipLaunchKernelGGL((gqa_merge_kernel<T, kGqaMaxDim>), grid, dim3(256), 0, st, a, tile_rows);
+  else
+    hipLaunchKernelGGL((gqa_merge_kernel<T, kGqaMaxMergeDim>), grid, dim3(256), 0, st, a, tile_rows);
   return hipGetLastError();
 }
 
@@ -511,6 +516,10 @@ hipError_t launch(const GqaArgs& a, int tile_rows, hipStream_t st) {
 int gqa_tile_rows(int dtype, int Dp, int Dvp, int rows) {
   if (rows <= kGqaSmallRows) return 16;
   return dtype == LLM_BF16 && std::max(Dp, Dvp) <= 128 ? 128 : 64;
+}
+
+hipError_t gqa_merge(int dtype, const GqaArgs& a, int tile_rows, hipStream_t st) {
+  return dtype == LLM_F32 ? merge<float>(a, tile_rows, st) : merge<__bf16>(a, tile_rows, st);
 }
 
 hipError_t gqa_attention(int dtype, const GqaArgs& a, int tile_rows, hipStream_t st) {

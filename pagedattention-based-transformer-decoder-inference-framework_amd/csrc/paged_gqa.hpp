@@ -32,6 +32,7 @@ struct GqaArgs {
   const void* q = nullptr;  // [tokens][H][Dp]
   void* out = nullptr;      // [tokens][ldo], head h's values at h * Dv
   int ldo = 0;
+  int ldh = 0;              // elements between the heads of out (0: Dv)
   const void* k_pool = nullptr;  // page [64][Dp]
   const void* v_pool = nullptr;  // page [Dvp][64] (mm.hpp v_page_slot)
   size_t page_stride = 0;        // bytes
@@ -54,5 +55,8 @@ int gqa_tile_rows(int dtype, int Dp, int Dvp, int rows);
 inline int gqa_part_dim(int Dv) { return (Dv + 15) / 16 * 16; }
 // One launch; every item was cut for tile_rows.
 hipError_t gqa_attention(int dtype, const GqaArgs& a, int tile_rows, hipStream_t st);
+// The merges of a launch that left partial states (gqa_attention does its own).
+constexpr int kGqaMaxMergeDim = 512;
+hipError_t gqa_merge(int dtype, const GqaArgs& a, int tile_rows, hipStream_t st);
 
 }  // namespace llm

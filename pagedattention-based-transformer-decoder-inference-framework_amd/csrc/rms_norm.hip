@@ -1,6 +1,7 @@
-// The residual stream between sublayers: add the normed sublayer output, add
-// the embedding where a repeated pass starts, norm for the next sublayer --
-// one launch, the row in registers.  Also the rotation angles of a step.
+// The residual stream (or streams) between sublayers: add the sublayer output,
+// normed or scaled, add the embedding where a repeated pass starts, norm for the
+// next sublayer -- one launch, the row in registers.  Also the rotation angles
+// of a step.
 #include "common.hpp"
 #include "rms_norm.hpp"
 
@@ -26,25 +27,40 @@ __device__ __forceinline__ float square_sum(f32x4 v) {
   return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
 }
 
-// THREADS lanes per row, NV float4 per lane
-template <typename T, int THREADS, int NV>
+// THREADS lanes per row, NV float4 per lane; SM: most streams (0: one residual)
+template <typename T, int THREADS, int NV, int SM>
 __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
+  constexpr int SN = SM > 0 ? SM : 1;
   __shared__ float sh[THREADS / 64];
+  __shared__ float coef[SN * SN + 2 * SN];  // mix, out, in
   const int i = blockIdx.x;
   const int m = a.rows ? a.rows[i] : i;
   const int nv = a.ldx >> 2;
-  float* xr = a.x + (size_t)m * a.ldx;
+  float* xr = a.x + (size_t)m * (SM > 0 ? a.streams : 1) * a.ldx;
   f32x4 x[NV];
   auto embed_at = [&](int c) {
     const uint2 e = *reinterpret_cast<const uint2*>(a.emb + (size_t)a.tok[m] * a.ldx + 4 * c);
     return f32x4{__builtin_bit_cast(float, e.x << 16), __builtin_bit_cast(float, e.x & 0xFFFF0000u),
-                 __builtin_bit_cast(float, e.y << 16), __builtin_bit_cast(float, e.y & 0xFFFF0000u)};
+                 __builtin_bit_cast(float, e.y << 16),
+                 __builtin_bit_cast(float, e.y & 0xFFFF0000u)} * a.emb_scale;
   };
+  if constexpr (SM == 0) {
 #pragma unroll
-  for (int j = 0; j < NV; ++j) {
-    const int c = threadIdx.x + j * THREADS;
-    x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    if (c < nv) x[j] = a.embed == 1 ? embed_at(c) : *reinterpret_cast<const f32x4*>(xr + 4 * c);
+    for (int j = 0; j < NV; ++j) {
+      const int c = threadIdx.x + j * THREADS;
+      x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (c < nv) x[j] = a.embed == 1 ? embed_at(c) : *reinterpret_cast<const f32x4*>(xr + 4 * c);
+    }
+  } else {
+    const int S = a.streams;
+    for (int k = threadIdx.x; k < S * S + 2 * S; k += THREADS) {
+      float v = 1.f;  // hc_in
+      if (k < S * S) v = a.y ? a.hc_mix[k] : k / S == k % S ? 1.f : 0.f;
+      else if (k < S * S + S) v = a.y ? a.hc_out[k - S * S] : 0.f;
+      else if (a.hc_in) v = a.hc_in[k - S * S - S];
+      coef[k] = v;
+    }
+    __syncthreads();
   }
   const float inv_w = 1.f / (float)a.width;
   // the norm weights fly while the rows are summed
@@ -56,8 +72,8 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
     if (c < nv && a.w_post) wpost[j] = *reinterpret_cast<const f32x4*>(a.w_post + 4 * c);
     if (c < nv && a.w_pre) wpre[j] = *reinterpret_cast<const f32x4*>(a.w_pre + 4 * c);
   }
-  if (a.w_post) {
-    f32x4 y[NV];
+  f32x4 y[NV];
+  if (a.y) {
     float ss = 0.f;
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
@@ -83,25 +99,69 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
       y[j] = s;
       ss += square_sum(s);
     }
-    const float r = 1.f / sqrtf(row_sum<THREADS>(ss, sh) * inv_w + a.eps);
+    if (a.w_post) {
+      const float r = 1.f / sqrtf(row_sum<THREADS>(ss, sh) * inv_w + a.eps);
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int c = threadIdx.x + j * THREADS;
-      if (c < nv) x[j] += y[j] * r * wpost[j];
+      for (int j = 0; j < NV; ++j) y[j] = y[j] * r * wpost[j];
     }
-  }
-  if (a.embed == 2) {
+    if (a.y_scale) {
 #pragma unroll
-    for (int j = 0; j < NV; ++j) {
-      const int c = threadIdx.x + j * THREADS;
-      if (c < nv) x[j] += embed_at(c);
+      for (int j = 0; j < NV; ++j) {
+        const int c = threadIdx.x + j * THREADS;
+        if (c < nv) y[j] *= *reinterpret_cast<const f32x4*>(a.y_scale + 4 * c);
+      }
     }
+  } else {
+#pragma unroll
+    for (int j = 0; j < NV; ++j) y[j] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
-  if ((a.w_post || a.embed) && !a.rows) {
+  if constexpr (SM == 0) {
+    if (a.y) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) x[j] += y[j];
+    }
+    if (a.embed == 2) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int c = threadIdx.x + j * THREADS;
+        if (c < nv) x[j] += embed_at(c);
+      }
+    }
+    if ((a.y || a.embed) && !a.rows) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int c = threadIdx.x + j * THREADS;
+        if (c < nv) *reinterpret_cast<f32x4*>(xr + 4 * c) = x[j];
+      }
+    }
+  } else {
+    // x[j] becomes u; the streams themselves pass through
+    const int S = a.streams;
+    const float *mix = coef, *out = coef + S * S, *in = out + S;
+    const bool store = (a.y || a.embed) && !a.rows;
 #pragma unroll
     for (int j = 0; j < NV; ++j) {
       const int c = threadIdx.x + j * THREADS;
-      if (c < nv) *reinterpret_cast<f32x4*>(xr + 4 * c) = x[j];
+      x[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+      if (c >= nv) continue;
+      f32x4 old[SN];
+      const f32x4 e = a.embed ? embed_at(c) : f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < SN; ++s)
+        if (s < S)
+          old[s] = a.embed == 1 ? e : *reinterpret_cast<const f32x4*>(xr + (size_t)s * a.ldx + 4 * c);
+#pragma unroll(SN <= 4 ? SN : 1)
+      for (int t = 0; t < SN; ++t) {
+        if (t >= S) break;
+        f32x4 v = out[t] * y[j];
+#pragma unroll
+        for (int s = 0; s < SN; ++s)
+          if (s < S) v += mix[s * S + t] * old[s];
+        if (a.embed == 2) v += e;
+        if (store) *reinterpret_cast<f32x4*>(xr + (size_t)t * a.ldx + 4 * c) = v;
+        x[j] += in[t] * v;
+      }
+      if (a.u) *reinterpret_cast<f32x4*>(a.u + (size_t)i * a.ldx + 4 * c) = x[j];
     }
   }
   if (!a.w_pre) return;
@@ -123,12 +183,12 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
   }
 }
 
-template <typename T>
+template <typename T, int SM>
 hipError_t launch_norm(const NormStep& a, hipStream_t st) {
   const dim3 grid(a.M);
   const int nv = a.ldx >> 2;
 #define LLM_NORM_GO(TH, NV)                                                           \
-  hipLaunchKernelGGL((norm_step_kernel<T, TH, NV>), grid, dim3(TH), 0, st, a);        \
+  hipLaunchKernelGGL((norm_step_kernel<T, TH, NV, SM>), grid, dim3(TH), 0, st, a);    \
   return hipGetLastError()
   if (nv <= 64) { LLM_NORM_GO(64, 1); }
   if (nv <= 128) { LLM_NORM_GO(64, 2); }
@@ -138,6 +198,13 @@ hipError_t launch_norm(const NormStep& a, hipStream_t st) {
   if (nv <= 2048) { LLM_NORM_GO(256, 8); }
 #undef LLM_NORM_GO
   return hipErrorInvalidValue;
+}
+
+template <typename T>
+hipError_t launch_norm(const NormStep& a, hipStream_t st) {
+  if (a.streams == 0) return launch_norm<T, 0>(a, st);
+  if (a.streams <= 4) return launch_norm<T, 4>(a, st);
+  return a.streams <= kMaxStreams ? launch_norm<T, kMaxStreams>(a, st) : hipErrorInvalidValue;
 }
 
 __global__ void rope_turns_kernel(const int32_t* __restrict__ pos, int M,

@@ -115,7 +115,7 @@ def create(lib, folder, **kw):
 
 def test_registry_lists_every_architecture(lib):
     assert lib.llm_model_architectures().decode().split(",") == ["CUDADecoder", "Gefarax",
-                                                                "INT8Decoder"]
+                                                                "INT8Decoder", "Nubosun"]
 
 
 def test_config_faults_are_named(lib, tmp_path):
