@@ -3,7 +3,7 @@
 
     python bench.py [--gpus N] [--steps K] [--warmup W] [--config c3|c2|c4|c5|c1]
     python -m torch.distributed.run --nproc-per-node N bench.py --gpus N ...
-    python bench.py --engine [small|large|all]   (bench_engine.py)
+    python bench.py --engine [small|large|all] [--engine-model gefarax|nubosun]   (bench_engine.py)
 
 Workload (default): INT8Decoder with 24 layers, 16 heads,
 head_dim 128 (hidden 2048, inter 8192, vocab 50257), a batch of 64 sequences,
@@ -514,8 +514,10 @@ def main():
                     help="sensitivity runs only: pages in allocation order instead of the "
                          "shuffled pool SURVEY §8d measures on")
     ap.add_argument("--engine", nargs="?", const="all", choices=["small", "large", "all"],
-                    help="instead of the decode benchmark: the layer-stack model (Gefarax) "
-                         "through the serving engine beside the FP16 decoder at equal size")
+                    help="instead of the decode benchmark: a layer-stack model through the "
+                         "serving engine beside the closest other model at equal size")
+    ap.add_argument("--engine-model", default="gefarax", choices=["gefarax", "nubosun"],
+                    help="--engine: Gefarax beside the FP16 decoder, or Nubosun beside Gefarax")
     ap.add_argument("--stub-step", action="store_true", help=argparse.SUPPRESS)
     ap.add_argument("--stub-fail-rank", type=int, default=-1, help=argparse.SUPPRESS)
     args = ap.parse_args()
@@ -526,7 +528,7 @@ def main():
         raise SystemExit("bench.py: --gpus must be >= 1")
     if args.engine:
         import bench_engine
-        print(json.dumps(bench_engine.run(args.engine, args.steps)), flush=True)
+        print(json.dumps(bench_engine.run(args.engine, args.steps, args.engine_model)), flush=True)
         return
     if "WORLD_SIZE" not in os.environ and args.gpus > 1:
         sys.exit(spawn_ranks(args.gpus, sys.argv[1:]))

@@ -133,7 +133,8 @@ def check_rows(got, want, dtype, close_calls=False):
 
 
 def logits(cfg, w, tokens):
-    return ls.forward(cfg, w, tokens)
+    f = ls.forward_streams if cfg["architecture"] == "Nubosun" else ls.forward
+    return f(cfg, w, tokens)
 
 
 def replay(eng, requests, schedule):
@@ -160,6 +161,48 @@ def replay(eng, requests, schedule):
     for s in seq.values():
         eng.close_seq(s)
     return {i: np.concatenate(v) for i, v in got.items() if v}
+
+
+def random_schedule(requests, live, seed):
+    """Mixed steps: some requests decode, others bring portions, some pause."""
+    rng = np.random.default_rng(seed)
+    waiting, left, running, steps = list(requests), {i: len(t) for i, t in requests.items()}, [], []
+    while waiting or running:
+        while waiting and len(running) < live:
+            running.append(waiting.pop(0))
+        step = []
+        for i in rng.permutation(running).tolist():
+            if rng.random() < 0.15 and len(running) > 1:
+                continue
+            n = int(rng.choice([1, 1, 1, 2, 3, 5, 16, 40, 64, 90]))
+            step.append((i, min(n, left[i])))
+        for i, n in step:
+            left[i] -= n
+            if left[i] == 0:
+                running.remove(i)
+        if step:
+            steps.append(step)
+    return steps
+
+
+def most_pages(requests, steps, page=64):
+    """The most pages the schedule's live requests hold at once."""
+    at, most = {}, 0
+    for step in steps:
+        for i, n in step:
+            at[i] = at.get(i, 0) + n
+        most = max(most, sum(-(-n // page) for n in at.values()))
+        for i, _ in step:
+            if at[i] == len(requests[i]):
+                del at[i]
+    return most
+
+
+def greedy(cfg, w, prompt, n):
+    t = list(prompt)
+    for _ in range(n):
+        t.append(int(logits(cfg, w, np.array(t))[-1].argmax()))
+    return t[len(prompt):]
 
 
 def portions(total, sizes):

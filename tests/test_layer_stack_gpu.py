@@ -203,28 +203,6 @@ def test_portions(serve, name, sizes, dtype):
     T.check_rows(got, T.logits(cfg, w, t), dtype)
 
 
-def random_schedule(requests, live, seed):
-    """Mixed steps: some requests decode, others bring portions, some pause."""
-    rng = np.random.default_rng(seed)
-    waiting, left, running, steps = list(requests), {i: len(t) for i, t in requests.items()}, [], []
-    while waiting or running:
-        while waiting and len(running) < live:
-            running.append(waiting.pop(0))
-        step = []
-        for i in rng.permutation(running).tolist():
-            if rng.random() < 0.15 and len(running) > 1:
-                continue
-            n = int(rng.choice([1, 1, 1, 2, 3, 5, 16, 40, 64, 90]))
-            step.append((i, min(n, left[i])))
-        for i, n in step:
-            left[i] -= n
-            if left[i] == 0:
-                running.remove(i)
-        if step:
-            steps.append(step)
-    return steps
-
-
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("name", sorted(MODELS))
 def test_mixed_batches_with_pages_and_slots_used_again(serve, name, dtype):
@@ -234,16 +212,8 @@ def test_mixed_batches_with_pages_and_slots_used_again(serve, name, dtype):
     w = model_weights(cfg, 19, dtype)
     req = {i: tokens(cfg, n, 20 + i) for i, n in
            enumerate([1, 70, 190, 5, 128, 64, 33, 150, 65, 2, 100, 129])}
-    steps = random_schedule(req, 4, 21)
-    # the most pages the schedule ever holds at once
-    at, most = {}, 0
-    for step in steps:
-        for i, n in step:
-            at[i] = at.get(i, 0) + n
-        most = max(most, sum(-(-n // 64) for n in at.values()))
-        for i, _ in step:
-            if at[i] == len(req[i]):
-                del at[i]
+    steps = T.random_schedule(req, 4, 21)
+    most = T.most_pages(req, steps)
     eng = serve(cfg, w, dtype, max_tokens=64 * most, max_seqs=4)
     free = eng.free_tokens
     got = T.replay(eng, req, steps)
@@ -380,13 +350,6 @@ def test_long_decoding_of_a_batch(serve, dtype):
         T.check_rows(got[i], T.logits(cfg, w, t), dtype)
 
 
-def greedy(cfg, w, prompt, n):
-    t = list(prompt)
-    for _ in range(n):
-        t.append(int(T.logits(cfg, w, np.array(t))[-1].argmax()))
-    return t[len(prompt):]
-
-
 def test_greedy_generation_through_the_scheduler(serve):
     """More requests than slots and than the pool holds at once."""
     cfg = MODELS["plain"]
@@ -395,7 +358,7 @@ def test_greedy_generation_through_the_scheduler(serve):
     eng = serve(cfg, w, max_seqs=3, max_tokens=64 * 6, max_step_tokens=48)
     out = eng.generate_batch(prompts, 12)
     for p, o in zip(prompts, out):
-        assert o == greedy(cfg, w, p, 12)
+        assert o == T.greedy(cfg, w, p, 12)
     assert eng.free_tokens == 64 * 6
     # the first generated id as the end of the request
     eos = out[1][3]
@@ -482,7 +445,7 @@ def test_generate_command(gpu, tmp_path):
                        capture_output=True, text=True, timeout=100)
     assert r.returncode == 0, r.stderr[-2000:]
     got = [[int(t) for t in x.split(",")] for x in r.stdout.split()]
-    assert got == [greedy(cfg, w, p, 6) for p in prompts]
+    assert got == [T.greedy(cfg, w, p, 6) for p in prompts]
 
 
 # ------------------------------------------- the other models behind the engine
