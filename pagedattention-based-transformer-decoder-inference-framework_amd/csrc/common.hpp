@@ -147,7 +147,12 @@ __device__ __forceinline__ void load_to_lds(const void* src, void* lds) {
   asm volatile("s_mov_b32 m0, %0\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off" ::"s"(at), "v"(src)
                : "memory", "m0");
 }
-__device__ __forceinline__ void wait_lds_loads() { asm volatile("s_waitcnt vmcnt(0)" ::: "memory"); }
+// The wait is the builtin: the compiler then knows that its own earlier loads are
+// there too and does not wait for them among the next stage's.
+__device__ __forceinline__ void wait_lds_loads() {
+  __builtin_amdgcn_s_waitcnt(0x0F70);  // vmcnt(0), the other counters at their most
+  asm volatile("" ::: "memory");
+}
 
 // Offset of activation element (m, k) in MFMA A-fragment order ("packed A"):
 // one contiguous 1 KiB block per (16-row tile, k-step), lane l of the block

@@ -57,6 +57,7 @@ constexpr int kDefaultStepTokens = 2048;
 constexpr int kMaxSplits = 64;
 constexpr int kTargetGroups = 512;   // workgroups an attention launch is split up to: 2 per CU
 constexpr int kMinSplitPages = 4;    // a page per wave
+constexpr int kMinLatentPages = 3;   // 16 rows x 4096 keys: 3 30.4 us, 4 35.3, 2 30.3 and a longer merge
 constexpr size_t kMaxGraphs = 256;   // decode shapes kept captured
 constexpr size_t kKeepBytes = (size_t)192 << 20;  // weights up to this stay in the Infinity Cache
 
@@ -478,7 +479,8 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
   const int want = (int)std::min<long long>(std::max<long long>(kTargetGroups / (tiles * p.G), 1), kMaxSplits);
   // single tokens share one split count, so a decode step keeps its launch
   // shape (and graph) while contexts grow
-  const int common = std::min(want, (max_pages + kMinSplitPages - 1) / kMinSplitPages);
+  const int least = p.latent ? kMinLatentPages : kMinSplitPages;
+  const int common = std::min(want, (max_pages + least - 1) / least);
   for (const StepSeq& s : batch) {
     const int rows = s.n * p.R;
     const int t0 = tok0;
@@ -489,7 +491,7 @@ void LayerStack::cut(const std::vector<StepSeq>& batch, Plan& p, bool big,
     for (int r0 = 0; r0 < rows; r0 += l.tile_rows) {
       const int last = s.p0 + (std::min(r0 + l.tile_rows, rows) - 1) / p.R;
       const int pages = last / kPageTokens + 1;
-      const int ns = big ? std::min(want, (pages + kMinSplitPages - 1) / kMinSplitPages) : common;
+      const int ns = big ? std::min(want, (pages + least - 1) / least) : common;
       for (int k = 0; k < ns; ++k)
         items.push_back(GqaItem{t0, slot, s.p0, r0, rows, (int)((long long)pages * k / ns),
                                 (int)((long long)pages * (k + 1) / ns), ns > 1 ? l.parts + k : -1});

@@ -157,9 +157,6 @@ __device__ __forceinline__ const char* a_lane(const KernelArgs& p, const Block<T
   return reinterpret_cast<const char*>(b.A + (size_t)m * b.lda) + 16 * (lane_id() >> 4);
 }
 
-// Where the column pair (n, n + 1) of row m goes, and what it still needs: found
-// before the sums are there, so the loads behind it (position, slot, page,
-// angle, assignment) overlap the weight stream.
 template <int EPI>
 struct History {};
 template <>
@@ -167,6 +164,71 @@ struct History<kConv> {  // of the pair's two channels: earlier inputs, taps, bi
   float v[2][kMmConvTaps - 1], w[2][kMmConvTaps], bias[2];
 };
 
+// What an epilogue needs of a row, and of a column pair (n, n + 1): found once
+// per row and column of a block's tiles.
+template <int EPI>
+struct RowOf {
+  static constexpr bool PAGED = EPI == kQkv || EPI == kExpand;
+  int m = -1;             // -1: no such row
+  int at = 0, entry = 0;  // paged: place in the page, page-table entry of head 0 (-1: none)
+  int pos = 0;
+
+  __device__ __forceinline__ RowOf() {}
+  template <typename T>
+  __device__ __forceinline__ RowOf(const KernelArgs& p, const Block<T>& b, int row) {
+    if (row >= b.M) return;
+    m = row;
+    if constexpr (PAGED) {
+      const MmQkv& e = p.q;
+      pos = e.pos[m];
+      const int tile = pos / kPageTokens;
+      at = pos % kPageTokens;
+      entry = tile < e.max_tiles ? e.slot[m] * e.G * e.max_tiles + tile : -1;
+    }
+  }
+};
+template <int EPI>
+struct ColOf {
+  int n = -1;  // -1: no such column
+  int part = 0, head = 0, d = 0;
+
+  __device__ __forceinline__ ColOf() {}
+  template <typename T>
+  __device__ __forceinline__ ColOf(const KernelArgs& p, const Block<T>& b, int col) {
+    if (col >= b.N) return;
+    n = col;
+    if constexpr (RowOf<EPI>::PAGED) {  // query, key, value
+      const MmQkv& e = p.q;
+      const int nq = e.H * e.D, nk = e.G * e.D;
+      part = n < nq ? 0 : n < nq + nk ? 1 : 2;
+      const int i = n - (part == 0 ? 0 : part == 1 ? nq : nq + nk), size = part == 2 ? e.Dv : e.D;
+      head = i / size;
+      d = i - head * size;
+    } else if constexpr (EPI == kLatent) {  // query, projected down
+      const MmLatent& e = p.lat;
+      const int hd = e.D + e.rot;
+      part = n >= e.H * hd;
+      if (part) {
+        d = n - e.H * hd;
+      } else {
+        head = n / hd;
+        d = n - head * hd;
+      }
+    }
+  }
+};
+
+template <typename T>
+__device__ __forceinline__ T* page_at(const MmQkv& e, void* pool, int entry, int head) {
+  const int page = e.table[(size_t)entry + (size_t)head * e.max_tiles];
+  return page >= 0 && page < e.num_pages
+             ? reinterpret_cast<T*>(static_cast<char*>(pool) + (size_t)page * e.page_stride)
+             : nullptr;
+}
+
+// Where a column pair of a row goes, and what it still needs: found before the
+// sums are there, so the loads behind it (page, angle, assignment) overlap the
+// weight stream.
 template <typename T, int EPI>
 struct Target {
   History<EPI> past;
@@ -174,8 +236,10 @@ struct Target {
   void* p1 = nullptr;  // the second column's place where it is not next to the first
   float cs = 1.f, sn = 0.f;  // rotation; kGroupOut: cs is the weight
 
-  __device__ __forceinline__ void find(const KernelArgs& p, const Block<T>& b, int m, int n) {
-    if (m >= b.M || n >= b.N) return;
+  __device__ __forceinline__ void find(const KernelArgs& p, const Block<T>& b, const RowOf<EPI>& r,
+                                       const ColOf<EPI>& c) {
+    const int m = r.m, n = c.n;
+    if (m < 0 || n < 0) return;
     if constexpr (EPI == kStore) {
       float* d = p.a.C + (size_t)m * p.a.ldc + n;
       p0 = d;
@@ -207,18 +271,16 @@ struct Target {
       p1 = n + 1 < b.N ? d + 1 : nullptr;
     } else if constexpr (EPI == kLatent) {
       const MmLatent& e = p.lat;
-      const int hd = e.D + e.rot;
-      if (n >= e.H * hd) {
-        p0 = e.down + (size_t)m * e.ldd + (n - e.H * hd);
-        return;
+      const bool turned = !c.part && c.d >= e.D;
+      T* q = static_cast<T*>(e.q) + ((size_t)m * e.H + c.head) * e.ldq + c.d;
+      float* down = e.down + (size_t)m * e.ldd + c.d;
+      p0 = c.part ? static_cast<void*>(down) : static_cast<void*>(q);
+      if (turned) {
+        const float2 t = e.turn[(size_t)m * (e.rot >> 1) + ((c.d - e.D) >> 1)];
+        cs = t.x;
+        sn = t.y;
+        p1 = static_cast<T*>(e.q_lat) + ((size_t)m * e.H + c.head) * e.ld_lat + e.lat_rot + (c.d - e.D);
       }
-      const int head = n / hd, d = n - head * hd;
-      p0 = static_cast<T*>(e.q) + ((size_t)m * e.H + head) * e.ldq + d;
-      if (d < e.D) return;
-      const float2 t = e.turn[(size_t)m * (e.rot >> 1) + ((d - e.D) >> 1)];
-      cs = t.x;
-      sn = t.y;
-      p1 = static_cast<T*>(e.q_lat) + ((size_t)m * e.H + head) * e.ld_lat + e.lat_rot + (d - e.D);
     } else if constexpr (EPI == kConv) {
       const MmConv& e = p.conv;
       if (n >= e.gate) {
@@ -244,30 +306,26 @@ struct Target {
       past.bias[1] = e.bias[n + 1];
     } else {
       const MmQkv& e = p.q;
-      const int nq = e.H * e.D, nk = e.G * e.D;
-      if (n < nq) {
-        const int head = n / e.D, d = n - head * e.D;
-        turn(e, m, d);
-        p0 = static_cast<T*>(e.q) + ((size_t)m * e.H + head) * e.Dp + d;
+      if (c.part == 0) {
+        turn(e, m, c.d);
+        p0 = static_cast<T*>(e.q) + ((size_t)m * e.H + c.head) * e.Dp + c.d;
         return;
       }
-      const int pos = e.pos[m], tile = pos / kPageTokens, at = pos % kPageTokens;
-      if (tile >= e.max_tiles) return;
-      const int32_t* table = e.table + (size_t)e.slot[m] * e.G * e.max_tiles + tile;
-      if (n < nq + nk) {
-        const int head = (n - nq) / e.D, d = n - nq - head * e.D;
-        turn(e, m, d);
-        char* page = page_of(e, e.k_pool, table[(size_t)head * e.max_tiles]);
-        if (page) p0 = reinterpret_cast<T*>(page) + (size_t)at * e.Dp + d;
+      if (r.entry < 0) return;
+      if (c.part == 1) {
+        turn(e, m, c.d);
+        T* page = page_at<T>(e, e.k_pool, r.entry, c.head);
+        if (page) p0 = page + (size_t)r.at * e.Dp + c.d;
         return;
       }
-      const int v = n - nq - nk, slot = v_page_slot(at, Kind<T>::BF16);
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        const int head = (v + j) / e.Dv, d = v + j - head * e.Dv;
-        if (head >= e.G) break;  // the second half of the last pair
-        char* page = page_of(e, e.v_pool, table[(size_t)head * e.max_tiles]);
-        if (page) (j ? p1 : p0) = reinterpret_cast<T*>(page) + (size_t)d * kPageTokens + slot;
+      const int slot = v_page_slot(r.at, Kind<T>::BF16);
+      T* page = page_at<T>(e, e.v_pool, r.entry, c.head);
+      if (page) p0 = page + (size_t)c.d * kPageTokens + slot;
+      if (c.d + 1 < e.Dv) {
+        if (page) p1 = page + (size_t)(c.d + 1) * kPageTokens + slot;
+      } else if (c.head + 1 < e.G) {  // (not the second half of the last pair)
+        page = page_at<T>(e, e.v_pool, r.entry, c.head + 1);
+        if (page) p1 = page + slot;
       }
     }
   }
@@ -349,28 +407,77 @@ struct Target {
     cs = t.x;
     sn = t.y;
   }
-  static __device__ __forceinline__ char* page_of(const MmQkv& e, void* pool, int page) {
-    return page >= 0 && page < e.num_pages ? static_cast<char*>(pool) + (size_t)page * e.page_stride
-                                           : nullptr;
+};
+
+// A column of 16 x 16 tiles of finished sums (tile i's rows m0 + 16 i .., columns
+// n0 ..) -> the epilogue, a column pair per lane.  Every lane of the wave takes
+// part; rows are what row_of() found for this lane.
+template <typename T, int EPI, int MT>
+struct TileRows {
+  RowOf<EPI> r[MT][2];
+  __device__ __forceinline__ TileRows(const KernelArgs& p, const Block<T>& b, int m0) {
+    const int lane = lane_id(), first = m0 + 4 * (lane >> 4) + (lane & 1 ? 2 : 0);
+#pragma unroll
+    for (int i = 0; i < MT; ++i)
+#pragma unroll
+      for (int k = 0; k < 2; ++k) r[i][k] = RowOf<EPI>(p, b, first + 16 * i + k);
   }
 };
 
-// One 16 x 16 tile of finished sums (rows m0.., columns n0..) -> the epilogue,
-// a column pair per lane.  Every lane of the wave takes part.
-template <typename T, int EPI>
-__device__ __forceinline__ void emit_tile(const KernelArgs& p, const Block<T>& b, f32x4 c, int m0,
-                                          int n0) {
+template <typename T, int EPI, int MT, int NT>
+__device__ __forceinline__ void emit_column(const KernelArgs& p, const Block<T>& b,
+                                            const TileRows<T, EPI, MT>& rows, const f32x4 (&acc)[MT][NT],
+                                            int j, int m0, int n0) {
   const int lane = lane_id();
-  f32x4 o;
-#pragma unroll
-  for (int r = 0; r < 4; ++r) o[r] = mov_dpp<0xB1>(c[r]);  // the neighbouring column
   const bool odd = lane & 1;
-  const int n = n0 + (lane & 14);
+  if constexpr (RowOf<EPI>::PAGED) {
+    // values lie token by token: a lane's four rows of its own column are one
+    // store where they are tokens 4 t .. 4 t + 3 of a sequence
+    if (n0 >= (p.q.H + p.q.G) * p.q.D) {
+      typedef T quad_t __attribute__((ext_vector_type(4)));
+      const ColOf<EPI> col(p, b, n0 + (lane & 15));
 #pragma unroll
-  for (int r = 0; r < 2; ++r) {
-    Target<T, EPI> t;
-    t.find(p, b, m0 + 4 * (lane >> 4) + (odd ? 2 : 0) + r, n);
-    t.put(p, b, n, odd ? o[2 + r] : c[r], odd ? c[2 + r] : o[r]);
+      for (int i = 0; i < MT; ++i) {
+        const int m = m0 + 16 * i + 4 * (lane >> 4);
+        const RowOf<EPI> lo(p, b, m), hi(p, b, m + 3);
+        if (lo.m < 0 || col.n < 0) continue;
+        if (hi.m >= 0 && (lo.at & 3) == 0 && hi.pos == lo.pos + 3 && hi.entry == lo.entry) {
+          if (lo.entry < 0) continue;
+          T* page = page_at<T>(p.q, p.q.v_pool, lo.entry, col.head);
+          if (!page) continue;
+          quad_t v;
+#pragma unroll
+          for (int r = 0; r < 4; ++r) v[r] = (T)acc[i][j][r];
+          *reinterpret_cast<quad_t*>(page + (size_t)col.d * kPageTokens +
+                                     v_page_slot(lo.at, Kind<T>::BF16)) = v;
+        } else {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            const RowOf<EPI> row(p, b, m + r);
+            if (row.m < 0 || row.entry < 0) continue;
+            T* page = page_at<T>(p.q, p.q.v_pool, row.entry, col.head);
+            if (page)
+              page[(size_t)col.d * kPageTokens + v_page_slot(row.at, Kind<T>::BF16)] = (T)acc[i][j][r];
+          }
+        }
+      }
+      return;
+    }
+  }
+  const int n = n0 + (lane & 14);
+  const ColOf<EPI> col(p, b, n);
+#pragma unroll
+  for (int i = 0; i < MT; ++i) {
+    const f32x4 c = acc[i][j];
+    f32x4 o;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) o[r] = mov_dpp<0xB1>(c[r]);  // the neighbouring column
+#pragma unroll
+    for (int r = 0; r < 2; ++r) {
+      Target<T, EPI> t;
+      t.find(p, b, rows.r[i][r], col);
+      t.put(p, b, n, odd ? o[2 + r] : c[r], odd ? c[2 + r] : o[r]);
+    }
   }
 }
 
@@ -449,8 +556,8 @@ __global__ __launch_bounds__(64 * WK, MT * NT == 1 ? 4 : 2) void mm_stream_kerne
   for (int e = 0; e < EPT; ++e) {
     const int pr = threadIdx.x + e * THREADS, t = pr >> 7;
     if (pr < PAIRS)
-      target[e].find(p, b, b.m0 + 16 * (t / NT) + ((pr >> 3) & 15),
-                     (nt0 + t % NT) * 16 + (pr & 7) * 2);
+      target[e].find(p, b, RowOf<EPI>(p, b, b.m0 + 16 * (t / NT) + ((pr >> 3) & 15)),
+                     ColOf<EPI>(p, b, (nt0 + t % NT) * 16 + (pr & 7) * 2));
   }
   if (ks0 < ks1) {
     for (int ks = ks0;;) {
@@ -551,11 +658,10 @@ __global__ __launch_bounds__(256, 2) void mm_block_kernel(KernelArgs p) {
     mul(st, 0);
     if (ks + 1 < b.KS) mul(st, 1);
   }
+  const int m0 = b.m0 + 16 * wm * MT;
+  const TileRows<T, EPI, MT> rows(p, b, m0);
 #pragma unroll
-  for (int i = 0; i < MT; ++i)
-#pragma unroll
-    for (int j = 0; j < NT; ++j)
-      emit_tile<T, EPI>(p, b, acc[i][j], b.m0 + 16 * (wm * MT + i), (nt0 + wn * NT + j) * 16);
+  for (int j = 0; j < NT; ++j) emit_column(p, b, rows, acc, j, m0, (nt0 + wn * NT + j) * 16);
 }
 
 template <int EPI>
@@ -591,6 +697,10 @@ hipError_t launch(const KernelArgs& p, hipStream_t st) {
   if (M <= 64)
     return ntiles * b16 < 256 ? stream<T, EPI, 1, 1>(p, b16, N, st)
                               : stream<T, EPI, 1, 2>(p, b16, N, st);
+  if constexpr (EPI == kSplit) {
+    // narrow products: all columns in two blocks, so a row is read twice
+    if (ntiles <= 10 && (M + 31) / 32 * 2 < 1024) return stream<T, EPI, 2, 5>(p, (M + 31) / 32, N, st);
+  }
   // prompt rows: blocks once there are enough of them, else 32-row streams
   const int n128 = (N + 127) / 128 * heads_of<EPI>(p);
   if ((M + 127) / 128 * n128 >= 256) return blocks<T, EPI, 8, 2>(p, (M + 127) / 128, N, st);

@@ -55,11 +55,11 @@ __device__ __forceinline__ f32x4 dot_step(u32x4 a, u32x4 b, f32x4 c) {
   }
 }
 
-// The rows one wave works on.  C: largest Dp / Dvp of the class (64, 128, 256).
-template <typename T, int C, int MT>
+// The rows one wave works on.  CK, CV: largest Dp and Dvp of the class.
+template <typename T, int CK, int CV, int MT>
 struct Rows {
   static constexpr int KSTEP = Att<T>::KSTEP, KT = Att<T>::KT, KEYS = 16 * KT;
-  static constexpr int NK = C / KSTEP, ND = C / 16;
+  static constexpr int NK = CK / KSTEP, ND = CV / 16;
   u32x4 q[MT][NK];
   f32x4 o[ND][MT];
   float m[MT], l[MT];
@@ -222,7 +222,7 @@ __device__ __forceinline__ int page_at(const GqaArgs& a, const int32_t* pt, int 
 
 template <typename T, int C>
 __global__ __launch_bounds__(64 * kWaves, C < 256 ? 2 : 1) void gqa_split_kernel(GqaArgs a) {
-  using RowsT = Rows<T, C, 1>;
+  using RowsT = Rows<T, C, C, 1>;
   constexpr int KSTEP = RowsT::KSTEP, KT = RowsT::KT, KEYS = RowsT::KEYS;
   constexpr int NK = RowsT::NK, ND = RowsT::ND;
   constexpr int BPP = kPageTokens / KEYS;
@@ -344,20 +344,22 @@ __global__ __launch_bounds__(64 * kWaves, C < 256 ? 2 : 1) void gqa_split_kernel
 }
 
 // Keys a stage of the row kernel holds: 32 KiB of K and V fragments at most.
-template <typename T, int C>
+template <typename T, int CK, int CV>
 constexpr int stage_keys() {
-  return (int)std::min<size_t>(kPageTokens, 32768 / (2 * C * sizeof(T)));
+  int n = kPageTokens;
+  while (n * (CK + CV) * (int)sizeof(T) > 32768) n /= 2;
+  return n;
 }
 
-template <typename T, int C, int MT>
+template <typename T, int CK, int CV, int MT>
 __global__ __launch_bounds__(64 * kWaves, 2) void gqa_rows_kernel(GqaArgs a) {
-  using RowsT = Rows<T, C, MT>;
+  using RowsT = Rows<T, CK, CV, MT>;
   constexpr int KSTEP = RowsT::KSTEP, KT = RowsT::KT, KEYS = RowsT::KEYS;
   constexpr int NK = RowsT::NK, ND = RowsT::ND;
-  constexpr int SK = stage_keys<T, C>(), SPP = kPageTokens / SK;
+  constexpr int SK = stage_keys<T, CK, CV>(), SPP = kPageTokens / SK;
   constexpr int FK = SK / 16 * NK, FV = SK / KEYS * ND, FW = (FK + FV) / kWaves;
   constexpr int TR = 16 * MT * kWaves;
-  static_assert(SK % KEYS == 0 && FK % FW == 0, "a wave loads K or V fragments, not both");
+  static_assert(SK % KEYS == 0 && (FK + FV) % kWaves == 0, "whole fragments per wave");
   __shared__ u32x4 lds[2][FK + FV][64];
 
   const int lane = lane_id(), w = wave_id_uniform();
@@ -493,9 +495,9 @@ hipError_t split(const GqaArgs& a, hipStream_t st) {
   return merge<T>(a, 16, st);
 }
 
-template <typename T, int C, int MT>
+template <typename T, int CK, int CV, int MT>
 hipError_t rows(const GqaArgs& a, hipStream_t st) {
-  hipLaunchKernelGGL((gqa_rows_kernel<T, C, MT>), dim3(a.n_items, a.G), dim3(64 * kWaves), 0, st, a);
+  hipLaunchKernelGGL((gqa_rows_kernel<T, CK, CV, MT>), dim3(a.n_items, a.G), dim3(64 * kWaves), 0, st, a);
   if (hipError_t e = hipGetLastError()) return e;
   return merge<T>(a, 16 * MT * kWaves, st);
 }
@@ -505,17 +507,21 @@ hipError_t launch(const GqaArgs& a, int tile_rows, hipStream_t st) {
   const int d = std::max(a.Dp, a.Dvp);
   if (tile_rows == 16)
     return d <= 64 ? split<T, 64>(a, st) : d <= 128 ? split<T, 128>(a, st) : split<T, 256>(a, st);
-  if (sizeof(T) == 2 && d <= 64) return rows<T, 64, sizeof(T) == 2 ? 2 : 1>(a, st);
-  if (sizeof(T) == 2 && d <= 128) return rows<T, 128, sizeof(T) == 2 ? 2 : 1>(a, st);
-  if (d <= 64) return rows<T, 64, 1>(a, st);
-  return d <= 128 ? rows<T, 128, 1>(a, st) : rows<T, 256, 1>(a, st);
+  if constexpr (sizeof(T) == 2) {
+    if (tile_rows == 128) {
+      if (d <= 64) return rows<T, 64, 64, 2>(a, st);
+      return d <= 128 ? rows<T, 128, 128, 2>(a, st) : rows<T, 192, 128, 2>(a, st);
+    }
+  }
+  if (d <= 64) return rows<T, 64, 64, 1>(a, st);
+  return d <= 128 ? rows<T, 128, 128, 1>(a, st) : rows<T, 256, 256, 1>(a, st);
 }
 
 }  // namespace
 
 int gqa_tile_rows(int dtype, int Dp, int Dvp, int rows) {
   if (rows <= kGqaSmallRows) return 16;
-  return dtype == LLM_BF16 && std::max(Dp, Dvp) <= 128 ? 128 : 64;
+  return dtype == LLM_BF16 && Dp <= 192 && Dvp <= 128 ? 128 : 64;
 }
 
 hipError_t gqa_merge(int dtype, const GqaArgs& a, int tile_rows, hipStream_t st) {

@@ -48,10 +48,14 @@ template <typename T, int NK, int NDW, int MT, int SK>
 __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1) void latent_kernel(GqaArgs a) {
   constexpr bool BF16 = sizeof(T) == 2;
   constexpr int KSTEP = BF16 ? 32 : 16, KT = BF16 ? 2 : 1;  // 16-key tiles per step of product 2
-  constexpr int KTS = SK / 16, NG = kWaves / MT, UW = (KTS + NG - 1) / NG;
+  // product 1: a row tile's NG waves share the key tiles, and where there are fewer
+  // of those, the row's k-steps (PARTS sums, added where they are read)
+  constexpr int KTS = SK / 16, NG = kWaves / MT;
+  constexpr int PARTS = NG > KTS ? NG / KTS : 1, UG = NG / PARTS, UW = KTS / UG, NKP = NK / PARTS;
+  static_assert(UG * PARTS == NG && UW * UG == KTS && NKP * PARTS == NK, "even shares");
   constexpr int SPP = kPageTokens / SK, FILL = (SK * 4 * NK + 255) / 256;
   __shared__ u32x4 stage[2][SK * 4 * NK];
-  __shared__ f32x4 score[MT][KTS][64];
+  __shared__ f32x4 score[MT][KTS][PARTS][64];
 
   const int lane = lane_id(), w = wave_id_uniform();
   const int g = lane >> 4, c = lane & 15;
@@ -81,18 +85,18 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
       if (q0 < SK * cpr) load_to_lds(src + from[i], &stage[buf][q0]);
     }
   };
-  auto page_of = [&](int s) {
-    const int tile = s / SPP;
-    int p = s < s1 && tile < a.max_tiles ? pt[tile] : -1;
-    p = p < a.num_pages ? p : -1;
+  // a stage's page: looked up a stage before it is asked for
+  auto lookup = [&](int s) { return pt[min(s / SPP, a.max_tiles - 1)]; };
+  auto page_of = [&](int s, int found) {
+    const int p = s < s1 && s / SPP < a.max_tiles && found < a.num_pages ? found : -1;
     return __builtin_amdgcn_readfirstlane(p);
   };
-  int page = page_of(s0), next = page_of(s0 + 1), buf = 0;
+  int page = page_of(s0, lookup(s0)), next = page_of(s0 + 1, lookup(s0 + 1)), buf = 0;
   issue(0, s0, page);
 
-  // product 1: this wave's row tile and key tiles u0, u0 + NG, ...
-  const int t1 = w % MT, u0 = w / MT;
-  u32x4 q[NK];
+  // this wave's row tile, key tiles u0, u0 + UG, ... and k-steps k1 ..
+  const int t1 = w % MT, u0 = w / MT % UG, part = w / MT / UG, k1 = part * NKP;
+  u32x4 q[NKP];
   {
     const int rr = 16 * t1 + c;
     const bool ok = rr < rows;
@@ -100,13 +104,14 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
     const T* qp = static_cast<const T*>(a.q) +
                   ((size_t)(it.tok0 + tok) * R + (row - tok * R)) * a.Dp + g * (KSTEP / 4);
 #pragma unroll
-    for (int k = 0; k < NK; ++k)
-      q[k] = ok && k * KSTEP < a.Dp ? *reinterpret_cast<const u32x4*>(qp + k * KSTEP)
-                                    : u32x4{0u, 0u, 0u, 0u};
+    for (int k = 0; k < NKP; ++k)  // (steps past the row meet zeros)
+      q[k] = ok && (k1 + k) * KSTEP < a.Dp
+                 ? *reinterpret_cast<const u32x4*>(qp + (k1 + k) * KSTEP)
+                 : u32x4{0u, 0u, 0u, 0u};
   }
   int turn1[UW];  // rotation of the key this lane reads in product 1
 #pragma unroll
-  for (int i = 0; i < UW; ++i) turn1[i] = (16 * (u0 + NG * i) + c) % cpr;
+  for (int i = 0; i < UW; ++i) turn1[i] = (16 * (u0 + UG * i) + c) % cpr;
   int turn2[KTS][BF16 ? 1 : 4];  // and in product 2
 #pragma unroll
   for (int u = 0; u < KTS; ++u) {
@@ -128,28 +133,30 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
     for (int n = 0; n < NDW; ++n) o[n][t] = f32x4{0.f, 0.f, 0.f, 0.f};
   }
   const float scale2 = a.scale * kLog2e;
+  const int last_tile = (a.Dv + 15) / 16 - 1;
 
   for (int s = s0; s < s1; ++s, buf ^= 1) {
-    const int after = page_of(s + 2);
     wait_lds_loads();
     __syncthreads();  // stage s has landed, the other buffer and the scores are read out
     issue(buf ^ 1, s + 1, next);
+    const int found = lookup(s + 2);
     const u32x4* st = stage[buf];
-    if (16 * t1 < rows) {
+    if (MT == 1 || 16 * t1 < rows) {
 #pragma unroll
       for (int i = 0; i < UW; ++i) {
-        const int u = u0 + NG * i;
-        if (u >= KTS) break;
+        const int u = u0 + UG * i;
         f32x4 d0 = {0.f, 0.f, 0.f, 0.f}, d1 = d0;
         const u32x4* row = st + (16 * u + c) * cpr;
+        u32x4 x[NKP];
 #pragma unroll
-        for (int k = 0; k < NK; ++k)
-          if (k * KSTEP < a.Dp) {
-            const u32x4 x = row[wrap(4 * k + g + turn1[i], cpr)];
-            if (k & 1) d1 = dot_step<T>(x, q[k], d1);
-            else d0 = dot_step<T>(x, q[k], d0);
-          }
-        score[t1][u][lane] = d0 + d1;
+        for (int k = 0; k < NKP; ++k)
+          x[k] = row[wrap(min(4 * (k1 + k) + g, cpr - 1) + turn1[i], cpr)];
+#pragma unroll
+        for (int k = 0; k < NKP; ++k) {
+          if (k & 1) d1 = dot_step<T>(x[k], q[k], d1);
+          else d0 = dot_step<T>(x[k], q[k], d0);
+        }
+        score[t1][u][part][lane] = d0 + d1;
       }
     }
     __syncthreads();
@@ -159,12 +166,15 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
       u32x4 hi[MT][KTS / KT], lo[MT][KTS / KT];
 #pragma unroll
       for (int t = 0; t < MT; ++t) {
-        if (16 * t >= rows) break;
+        if (t > 0 && 16 * t >= rows) break;
         f32x4 x[KTS];
         float mloc = kNegSentinel;
 #pragma unroll
         for (int u = 0; u < KTS; ++u) {
-          x[u] = score[t][u][lane] * scale2;
+          x[u] = score[t][u][0][lane];
+#pragma unroll
+          for (int i = 1; i < PARTS; ++i) x[u] += score[t][u][i][lane];
+          x[u] *= scale2;
           if (mask || 16 * t + 16 > rows) {
 #pragma unroll
             for (int r = 0; r < 4; ++r)
@@ -209,11 +219,11 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
       }
 #pragma unroll
       for (int b = 0; b < KTS / KT; ++b) {
+        u32x4 v[NDW];
 #pragma unroll
         for (int n = 0; n < NDW; ++n) {
-          const int tile = w + kWaves * n;
-          if (16 * tile >= a.Dv) break;
-          u32x4 v;
+          // (tiles past the latent repeat the last one, nobody reads their sums)
+          const int tile = min(w + kWaves * n, last_tile);
           if constexpr (BF16) {
             // lane 4 q + p of 16 addresses key 4 g + q, dims 4 p ..; it gets keys
             // 4 g .. 4 g + 3 of dim `lane`
@@ -227,8 +237,8 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
               half[j] = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                   (__attribute__((address_space(3))) s16x4*)at);
             }
-            v = __builtin_bit_cast(u32x4, s16x8{half[0][0], half[0][1], half[0][2], half[0][3],
-                                                half[1][0], half[1][1], half[1][2], half[1][3]});
+            v[n] = __builtin_bit_cast(u32x4, s16x8{half[0][0], half[0][1], half[0][2], half[0][3],
+                                                   half[1][0], half[1][1], half[1][2], half[1][3]});
           } else {
             const int d = 16 * tile + c;
             f32x4 f;
@@ -238,19 +248,22 @@ __global__ __launch_bounds__(64 * kWaves, sizeof(T) == 2 && NK * MT < 72 ? 2 : 1
               f[j] = reinterpret_cast<const float*>(
                   st + key * cpr + wrap((d >> 2) + turn2[b][j], cpr))[d & 3];
             }
-            v = __builtin_bit_cast(u32x4, f);
+            v[n] = __builtin_bit_cast(u32x4, f);
           }
+        }
 #pragma unroll
-          for (int t = 0; t < MT; ++t) {
-            if (16 * t >= rows) break;
-            o[n][t] = dot_step<T>(v, hi[t][b], o[n][t]);
-            if constexpr (BF16) o[n][t] = dot_step<T>(v, lo[t][b], o[n][t]);
+        for (int t = 0; t < MT; ++t) {
+          if (t > 0 && 16 * t >= rows) break;
+#pragma unroll
+          for (int n = 0; n < NDW; ++n) {
+            o[n][t] = dot_step<T>(v[n], hi[t][b], o[n][t]);
+            if constexpr (BF16) o[n][t] = dot_step<T>(v[n], lo[t][b], o[n][t]);
           }
         }
       }
     }
     page = next;
-    next = after;
+    next = page_of(s + 2, found);
   }
 
 #pragma unroll
@@ -329,32 +342,46 @@ __device__ __forceinline__ T* row_of(const MmPageRows& r, int pos, int slot) {
 
 // a wave per token
 template <typename T>
-__global__ __launch_bounds__(256) void append_kernel(LatentAppend a) {
+__global__ __launch_bounds__(64) void append_kernel(LatentAppend a) {
   constexpr int NV = kLatentMaxRank / 64;
-  const int mrow = (int)blockIdx.x * 4 + wave_id_uniform(), lane = lane_id();
-  if (mrow >= a.M) return;
+  const int mrow = blockIdx.x, lane = lane_id();
   const float* src = a.down + (size_t)mrow * a.ldd;
-  T* dst = row_of<T>(a.page, a.page.pos[mrow], a.page.slot[mrow]);
-  if (!dst) return;
-  float v[NV], ss = 0.f;
+  const int pos = a.page.pos[mrow], slot = a.page.slot[mrow];
+  // everything that does not hang on the page is on its way before it is known
+  float v[NV], w[NV], ss = 0.f;
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
-    const int d = lane + 64 * j;
-    v[j] = d < a.rank ? src[d] : 0.f;
+    const int d = min(lane + 64 * j, a.rank - 1);
+    v[j] = src[d];
+    w[j] = a.w[d];
+  }
+  const int pairs = a.rot / 2;
+  float2 t = {1.f, 0.f}, k = {0.f, 0.f};
+  if (lane < pairs) {
+    t = a.turn[(size_t)mrow * pairs + lane];
+    k = *reinterpret_cast<const float2*>(src + a.rot_at + 2 * lane);
+  }
+  T* dst = row_of<T>(a.page, pos, slot);
+#pragma unroll
+  for (int j = 0; j < NV; ++j) {
+    if (lane + 64 * j >= a.rank) v[j] = 0.f;
     ss += v[j] * v[j];
   }
   const float r = 1.f / sqrtf(wave_sum(ss) / (float)a.rank + a.eps);
+  if (!dst) return;
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int d = lane + 64 * j;
-    if (d < a.rank) dst[d] = (T)(v[j] * r * a.w[d]);
+    if (d < a.rank) dst[d] = (T)(v[j] * r * w[j]);
   }
   T* rot = dst + latent_rot_at(a.rank);
-  for (int i = lane; i < a.rot / 2; i += 64) {
-    const float2 t = a.turn[(size_t)mrow * (a.rot / 2) + i];
-    const float x = src[a.rot_at + 2 * i], y = src[a.rot_at + 2 * i + 1];
-    rot[2 * i] = (T)(x * t.x - y * t.y);
-    rot[2 * i + 1] = (T)(y * t.x + x * t.y);
+  for (int i = lane; i < pairs; i += 64) {
+    if (i != lane) {
+      t = a.turn[(size_t)mrow * pairs + i];
+      k = *reinterpret_cast<const float2*>(src + a.rot_at + 2 * i);
+    }
+    rot[2 * i] = (T)(k.x * t.x - k.y * t.y);
+    rot[2 * i + 1] = (T)(k.y * t.x + k.x * t.y);
   }
 }
 
@@ -383,9 +410,8 @@ hipError_t latent_attention(int dtype, const GqaArgs& a, int tile_rows, hipStrea
 
 hipError_t latent_append(int dtype, const LatentAppend& a, hipStream_t st) {
   if (a.M <= 0) return hipSuccess;
-  const dim3 grid((a.M + 3) / 4);
-  if (dtype == LLM_F32) hipLaunchKernelGGL(append_kernel<float>, grid, dim3(256), 0, st, a);
-  else hipLaunchKernelGGL(append_kernel<__bf16>, grid, dim3(256), 0, st, a);
+  if (dtype == LLM_F32) hipLaunchKernelGGL(append_kernel<float>, dim3(a.M), dim3(64), 0, st, a);
+  else hipLaunchKernelGGL(append_kernel<__bf16>, dim3(a.M), dim3(64), 0, st, a);
   return hipGetLastError();
 }
 

@@ -38,6 +38,9 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
   const int nv = a.ldx >> 2;
   float* xr = a.x + (size_t)m * (SM > 0 ? a.streams : 1) * a.ldx;
   f32x4 x[NV];
+  // up to 4 streams fly with the other loads; more are read where they are mixed
+  constexpr bool EARLY = SM > 0 && SM <= 4 && NV * SM <= 16;
+  f32x4 early[EARLY ? NV : 1][SN];
   auto embed_at = [&](int c) {
     const uint2 e = *reinterpret_cast<const uint2*>(a.emb + (size_t)a.tok[m] * a.ldx + 4 * c);
     return f32x4{__builtin_bit_cast(float, e.x << 16), __builtin_bit_cast(float, e.x & 0xFFFF0000u),
@@ -53,6 +56,17 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
     }
   } else {
     const int S = a.streams;
+    if constexpr (EARLY) {
+#pragma unroll
+      for (int j = 0; j < NV; ++j) {
+        const int c = min((int)threadIdx.x + j * THREADS, nv - 1);
+#pragma unroll
+        for (int s = 0; s < SN; ++s)
+          early[j][s] = a.embed == 1 ? embed_at(c)
+                                     : *reinterpret_cast<const f32x4*>(
+                                           xr + (size_t)min(s, S - 1) * a.ldx + 4 * c);
+      }
+    }
     for (int k = threadIdx.x; k < S * S + 2 * S; k += THREADS) {
       float v = 1.f;  // hc_in
       if (k < S * S) v = a.y ? a.hc_mix[k] : k / S == k % S ? 1.f : 0.f;
@@ -60,15 +74,16 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
       else if (a.hc_in) v = a.hc_in[k - S * S - S];
       coef[k] = v;
     }
-    __syncthreads();
   }
   const float inv_w = 1.f / (float)a.width;
   // the norm weights fly while the rows are summed
-  f32x4 wpost[NV], wpre[NV];
+  f32x4 wpost[NV], wpre[NV], scale[NV];
 #pragma unroll
   for (int j = 0; j < NV; ++j) {
     const int c = threadIdx.x + j * THREADS;
     wpost[j] = wpre[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    scale[j] = f32x4{1.f, 1.f, 1.f, 1.f};
+    if (c < nv && a.y_scale) scale[j] = *reinterpret_cast<const f32x4*>(a.y_scale + 4 * c);
     if (c < nv && a.w_post) wpost[j] = *reinterpret_cast<const f32x4*>(a.w_post + 4 * c);
     if (c < nv && a.w_pre) wpre[j] = *reinterpret_cast<const f32x4*>(a.w_pre + 4 * c);
   }
@@ -106,10 +121,7 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
     }
     if (a.y_scale) {
 #pragma unroll
-      for (int j = 0; j < NV; ++j) {
-        const int c = threadIdx.x + j * THREADS;
-        if (c < nv) y[j] *= *reinterpret_cast<const f32x4*>(a.y_scale + 4 * c);
-      }
+      for (int j = 0; j < NV; ++j) y[j] *= scale[j];
     }
   } else {
 #pragma unroll
@@ -136,6 +148,7 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
     }
   } else {
     // x[j] becomes u; the streams themselves pass through
+    __syncthreads();  // coef
     const int S = a.streams;
     const float *mix = coef, *out = coef + S * S, *in = out + S;
     const bool store = (a.y || a.embed) && !a.rows;
@@ -148,9 +161,10 @@ __global__ __launch_bounds__(THREADS) void norm_step_kernel(NormStep a) {
       const f32x4 e = a.embed ? embed_at(c) : f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
       for (int s = 0; s < SN; ++s)
-        if (s < S)
+        if constexpr (EARLY) old[s] = early[j][s];
+        else if (s < S)
           old[s] = a.embed == 1 ? e : *reinterpret_cast<const f32x4*>(xr + (size_t)s * a.ldx + 4 * c);
-#pragma unroll(SN <= 4 ? SN : 1)
+#pragma unroll SN <= 4 ? SN : 1
       for (int t = 0; t < SN; ++t) {
         if (t >= S) break;
         f32x4 v = out[t] * y[j];
@@ -190,6 +204,11 @@ hipError_t launch_norm(const NormStep& a, hipStream_t st) {
 #define LLM_NORM_GO(TH, NV)                                                           \
   hipLaunchKernelGGL((norm_step_kernel<T, TH, NV, SM>), grid, dim3(TH), 0, st, a);    \
   return hipGetLastError()
+  if (SM > 0 && a.M <= 256 && nv > 64) {  // few rows of several streams: a lane per column
+    if (nv <= 256) { LLM_NORM_GO(256, 1); }
+    if (nv <= 512) { LLM_NORM_GO(512, 1); }
+    if (nv <= 1024) { LLM_NORM_GO(1024, 1); }
+  }
   if (nv <= 64) { LLM_NORM_GO(64, 1); }
   if (nv <= 128) { LLM_NORM_GO(64, 2); }
   if (nv <= 256) { LLM_NORM_GO(256, 1); }

@@ -60,9 +60,9 @@ def test_streams(serve, streams, dtype):  # noqa: F811
         assert np.median(T.row_error(T.logits(cfg, turned, t), T.logits(cfg, w, t))) > 0.01
 
 
-def test_wide_residual(serve):  # noqa: F811
-    for width in (264, 700, 1100, 2500):
-        cfg = N.config([(N.mamba(inner=20), N.dense(ff=10))], width=width, vocab=40)
+def test_residual_widths(serve):  # noqa: F811
+    for width in (37, 264, 700, 1101, 2500):
+        cfg = N.config([(N.mamba(inner=20), N.dense(ff=10))], width=width, vocab=41)
         w = N.weights(cfg, 5)
         t = tokens(cfg, 20, 6)
         T.check_rows(run_whole(serve(cfg, w, name=f"w{width}"), t), T.logits(cfg, w, t), "float32")
