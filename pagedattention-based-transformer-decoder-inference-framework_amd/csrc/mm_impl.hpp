@@ -74,7 +74,24 @@ __device__ __forceinline__ float glu(float gate, float up, const GluParams& p) {
   return g / (1.f + expf(-p.alpha * g)) * (u + p.up_bias);
 }
 
-__device__ __forceinline__ float softplus(float v) { return v > 20.f ? v : log1pf(expf(v)); }
+// log(1 + e^v) = max(v, 0) + log1p(e), e = e^-|v|; log1p(e) = 2 atanh(s) with
+// s = e / (2 + e) <= 1/3, whose series needs no case for small or large v
+__device__ __forceinline__ float softplus(float v) {
+  const float a = -fabsf(v), t = a * kLog2e;
+  const float lo = fmaf(a, kLog2e, -t);  // what rounding took from the exponent
+  const float p = __builtin_amdgcn_exp2f(t);
+  const float e = fmaf(p, lo * 0.6931472f, p);
+  const float s = e * __builtin_amdgcn_rcpf(2.f + e), q = s * s;
+  float r = 1.f / 15.f;
+  r = fmaf(r, q, 1.f / 13.f);
+  r = fmaf(r, q, 1.f / 11.f);
+  r = fmaf(r, q, 1.f / 9.f);
+  r = fmaf(r, q, 1.f / 7.f);
+  r = fmaf(r, q, 1.f / 5.f);
+  r = fmaf(r, q, 1.f / 3.f);
+  r = fmaf(r, q, 1.f);
+  return fmaxf(v, 0.f) + 2.f * s * r;
+}
 
 template <typename T>
 __device__ __forceinline__ void put_pair(T* p, float v0, float v1) {
@@ -687,16 +704,33 @@ template <typename T, int EPI>
 hipError_t launch(const KernelArgs& p, hipStream_t st) {
   const int M = p.a.M, N = p.a.N;
   const int ntiles = (N + 15) / 16;
-  // rows in blocks of 16 (the weights of the later blocks come from L2): 64 x
-  // 2560 x 2048 10.8 us, against 12.8 in blocks of 32 and 13.8 in one of 64
-  const int b16 = (M + 15) / 16;
   if (M <= 16) return stream<T, EPI, 1, 1>(p, 1, N, st);
-  // two column tiles per block once that still fills the chip
-  if (M <= 64 && ntiles >= 512)
-    return M <= 32 ? stream<T, EPI, 2, 2>(p, 1, N, st) : stream<T, EPI, 4, 2>(p, 1, N, st);
-  if (M <= 64)
-    return ntiles * b16 < 256 ? stream<T, EPI, 1, 1>(p, b16, N, st)
-                              : stream<T, EPI, 1, 2>(p, b16, N, st);
+  if (M <= 64) {
+    // The form with the fewest rounds of workgroups over the chip, a round priced
+    // by its column tiles and the rows it reads: 64 x 12288 x 2048 17.4 us as 4 x 3
+    // tiles (one round) against 25.9 as 4 x 2, 64 x 8192 14.5 as 4 x 2 against 16.1.
+    struct Form {
+      int mt, nt;
+      float rows;
+      hipError_t (*go)(const KernelArgs&, int, int, hipStream_t);
+    };
+    static constexpr Form forms[] = {{1, 1, 0.5f, stream<T, EPI, 1, 1>}, {1, 2, 0.5f, stream<T, EPI, 1, 2>},
+                                     {2, 2, 1.5f, stream<T, EPI, 2, 2>}, {2, 3, 1.5f, stream<T, EPI, 2, 3>},
+                                     {4, 2, 3.f, stream<T, EPI, 4, 2>},  {4, 3, 3.f, stream<T, EPI, 4, 3>}};
+    const Form* best = nullptr;
+    int row_blocks = 0;
+    float least = 0.f;
+    for (const Form& f : forms) {
+      const int rb = (M + 16 * f.mt - 1) / (16 * f.mt);
+      const int groups = (ntiles + f.nt - 1) / f.nt * rb * heads_of<EPI>(p);
+      const float cost = (float)((groups + 255) / 256) * ((float)f.nt + f.rows);
+      if (best && cost >= least) continue;
+      best = &f;
+      least = cost;
+      row_blocks = rb;
+    }
+    return best->go(p, row_blocks, N, st);
+  }
   if constexpr (EPI == kSplit) {
     // narrow products: all columns in two blocks, so a row is read twice
     if (ntiles <= 10 && (M + 31) / 32 * 2 < 1024) return stream<T, EPI, 2, 5>(p, (M + 31) / 32, N, st);

@@ -16,7 +16,10 @@ constexpr int kThreads = 256;
 
 constexpr int chunk_of(int padded_state) { return std::min(64, 4096 / padded_state); }
 
-__device__ __forceinline__ float silu(float v) { return v / (1.f + expf(-v)); }
+// within 3 ulp: exp2 and the reciprocal are the hardware's
+__device__ __forceinline__ float silu(float v) {
+  return v * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-kLog2e * v));
+}
 
 enum Pass { kEmit, kChunk };
 
@@ -166,46 +169,83 @@ __global__ __launch_bounds__(kThreads) void scan_carry_kernel(ScanArgs a,
   }
 }
 
-// Two channels per lane, RB rows; rows of a block come from the cache lines the
-// block has just read.
-template <typename T>
+// Four channels per lane, RB rows.  TAPS (0: any number): blocks whose rows and
+// their past are one sequence's rows of this batch, nearly all of a prompt, read
+// each row once.
+template <typename T, int TAPS>
 __global__ __launch_bounds__(kThreads) void conv_kernel(ConvArgs a) {
-  typedef T pair_t __attribute__((ext_vector_type(2)));
+  typedef T quad_t __attribute__((ext_vector_type(4)));
   constexpr int RB = 8;
-  const int c = 2 * ((int)blockIdx.y * kThreads + threadIdx.x);
+  const int c = 4 * ((int)blockIdx.y * kThreads + threadIdx.x);
   if (c >= a.channels) return;
   const int m0 = (int)blockIdx.x * RB;
-  const float2 bias = *reinterpret_cast<const float2*>(a.bias + c);
-  float2 acc[RB];
+  const f32x4 bias = *reinterpret_cast<const f32x4*>(a.bias + c);
+  f32x4 acc[RB];
 #pragma unroll
   for (int r = 0; r < RB; ++r) acc[r] = bias;
-  for (int k = 0; k < a.taps; ++k) {
-    const float2 w = *reinterpret_cast<const float2*>(a.w + (size_t)k * a.ldc + c);
-    const int back = a.taps - 1 - k;
+  bool plain = false;
+  if constexpr (TAPS > 0) {
+    plain = m0 + RB <= a.M && a.seq0[min(m0 + RB, a.M) - 1] <= m0 - (TAPS - 1);
+    if (plain) {
+      quad_t v[RB + TAPS - 1];
+      const T* src = static_cast<const T*>(a.in) + (size_t)(m0 - (TAPS - 1)) * a.ld_in + c;
 #pragma unroll
-    for (int r = 0; r < RB; ++r) {
-      const int m = m0 + r;
-      if (m >= a.M) break;
-      const T* src = nullptr;
-      if (m - back >= a.seq0[m])
-        src = static_cast<const T*>(a.in) + (size_t)(m - back) * a.ld_in + c;
-      else if (a.pos[m] >= back)  // entry taps - 1 is the portion's first row
-        src = static_cast<const T*>(a.history) +
-              ((size_t)a.slot[m] * (a.taps - 1) + (m - back - a.seq0[m] + a.taps - 1)) * a.ldc + c;
-      if (!src) continue;
-      const pair_t v = *reinterpret_cast<const pair_t*>(src);
-      acc[r].x += w.x * (float)v[0];
-      acc[r].y += w.y * (float)v[1];
+      for (int r = 0; r < RB + TAPS - 1; ++r)
+        v[r] = *reinterpret_cast<const quad_t*>(src + (size_t)r * a.ld_in);
+#pragma unroll
+      for (int k = 0; k < TAPS; ++k) {
+        const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + (size_t)k * a.ldc + c);
+#pragma unroll
+        for (int r = 0; r < RB; ++r)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) acc[r][e] += w[e] * (float)v[r + k][e];
+      }
+    }
+  }
+  if (!plain) {
+    for (int k = 0; k < a.taps; ++k) {
+      const f32x4 w = *reinterpret_cast<const f32x4*>(a.w + (size_t)k * a.ldc + c);
+      const int back = a.taps - 1 - k;
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        const int m = m0 + r;
+        if (m >= a.M) break;
+        const T* src = nullptr;
+        if (m - back >= a.seq0[m])
+          src = static_cast<const T*>(a.in) + (size_t)(m - back) * a.ld_in + c;
+        else if (a.pos[m] >= back)  // entry taps - 1 is the portion's first row
+          src = static_cast<const T*>(a.history) +
+                ((size_t)a.slot[m] * (a.taps - 1) + (m - back - a.seq0[m] + a.taps - 1)) * a.ldc + c;
+        if (!src) continue;
+        const quad_t v = *reinterpret_cast<const quad_t*>(src);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) acc[r][e] += w[e] * (float)v[e];
+      }
     }
   }
 #pragma unroll
   for (int r = 0; r < RB; ++r) {
     if (m0 + r >= a.M) break;
-    pair_t v;
-    v[0] = (T)silu(acc[r].x);
-    v[1] = (T)silu(acc[r].y);
-    *reinterpret_cast<pair_t*>(static_cast<T*>(a.x) + (size_t)(m0 + r) * a.ldx + c) = v;
+    quad_t v;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] = (T)silu(acc[r][e]);
+    *reinterpret_cast<quad_t*>(static_cast<T*>(a.x) + (size_t)(m0 + r) * a.ldx + c) = v;
   }
+}
+
+template <typename T>
+hipError_t conv(const ConvArgs& a, hipStream_t st) {
+  const dim3 grid((a.M + 7) / 8, (a.channels + 4 * kThreads - 1) / (4 * kThreads));
+#define LLM_CONV_GO(TAPS) \
+  hipLaunchKernelGGL((conv_kernel<T, TAPS>), grid, dim3(kThreads), 0, st, a)
+  switch (a.taps) {
+    case 2: LLM_CONV_GO(2); break;
+    case 3: LLM_CONV_GO(3); break;
+    case 4: LLM_CONV_GO(4); break;
+    default: LLM_CONV_GO(0);
+  }
+#undef LLM_CONV_GO
+  return hipGetLastError();
 }
 
 template <typename T, int NS, int SP, int PASS>
@@ -258,12 +298,7 @@ hipError_t scan_carry(const ScanArgs& a, const ScanCarry* seqs, int n, hipStream
 
 hipError_t causal_conv(int dtype, const ConvArgs& a, hipStream_t st) {
   if (a.M <= 0) return hipSuccess;
-  const dim3 grid((a.M + 7) / 8, (a.channels + 2 * kThreads - 1) / (2 * kThreads));
-  if (dtype == LLM_F32)
-    hipLaunchKernelGGL(conv_kernel<float>, grid, dim3(kThreads), 0, st, a);
-  else
-    hipLaunchKernelGGL(conv_kernel<__bf16>, grid, dim3(kThreads), 0, st, a);
-  return hipGetLastError();
+  return dtype == LLM_F32 ? conv<float>(a, st) : conv<__bf16>(a, st);
 }
 
 }  // namespace llm

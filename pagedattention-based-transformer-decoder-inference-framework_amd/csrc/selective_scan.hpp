@@ -33,7 +33,7 @@ struct ScanCarry {
 
 struct ScanArgs {
   int inner = 0, state = 0;
-  int ldc = 0;                // channels per row of A, state, history and parts (even)
+  int ldc = 0;                // channels per row of A, state, history and parts (a multiple of 4)
   const void* x = nullptr;    // [M][ldx] after the convolution
   int ldx = 0;
   const float* dt = nullptr;  // [M][ldt]

@@ -433,6 +433,44 @@ def test_decoding_of_many(serve, batch):  # noqa: F811
         T.check_rows(got[i], T.logits(cfg, w, t), "float32")
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("vocab,ff,inner", [(33001, 6144, 8192), (12288, 4096, 6144), (8200, 3100, 4100)])
+def test_wide_products(serve, vocab, ff, inner, dtype):  # noqa: F811
+    """Few rows against many columns: every tile form of the row counts up to 64,
+    as portions and as decoded batches."""
+    cfg = N.config([(N.mamba(inner=inner, state=2), N.dense(ff=ff)),
+                    (N.latent(heads=40, dim=90, rot=8, vdim=8, rank=16), None)],
+                   width=40, vocab=vocab, streams=2)
+    w = N.weights(cfg, 44)
+    eng = serve(cfg, w, dtype, max_seqs=40, max_tokens=64 * 40)
+    for n in (16, 30, 47, 64):
+        t = tokens(cfg, n, n)
+        T.check_rows(run_whole(eng, t), T.logits(cfg, w, t), dtype)
+    req = {i: tokens(cfg, 3, i) for i in range(40)}
+    rows = (range(40), range(25), range(40), range(25, 40))
+    got = T.replay(eng, req, [[(i, 1) for i in r] for r in rows])
+    for i, t in req.items():
+        T.check_rows(got[i], T.logits(cfg, w, t), dtype)
+
+
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_long_prompts_of_wide_layers(serve, dtype):  # noqa: F811
+    """Every product in its prompt form, alone and beside single tokens; expanded
+    keys of several portions in one step, over pages that are not whole."""
+    cfg = N.config([(N.mamba(inner=4100, state=2), N.dense(ff=4096)),
+                    (N.latent(heads=40, dim=160, rot=8, vdim=24, rank=128), None)],
+                   width=40, vocab=200, streams=2)
+    w = N.weights(cfg, 46)
+    eng = serve(cfg, w, dtype, max_seqs=4, max_tokens=64 * 60)
+    req = {i: tokens(cfg, n, n) for i, n in enumerate((1030, 901, 400, 70))}
+    want = {i: T.logits(cfg, w, t) for i, t in req.items()}
+    T.check_rows(run_whole(eng, req[0]), want[0], dtype)
+    got = T.replay(eng, req, [[(2, 30), (0, 355), (3, 69), (1, 401)], [(1, 331), (3, 1), (0, 330), (2, 370)],
+                              [(0, 1), (1, 1)], [(1, 168), (0, 344)]])
+    for i in req:
+        T.check_rows(got[i], want[i], dtype)
+
+
 def test_greedy_generation_through_the_scheduler(serve):  # noqa: F811
     cfg = MODELS["plain"]
     w = N.weights(cfg, 45)
